@@ -70,12 +70,40 @@ SYMBOLS = {
     "onebit_train_backward": (_int, [_vp] * 13 + [ctypes.c_size_t, _i64, _i64, _i64, _int, _vp]),
 }
 
+# libonebit_hybrid.so (include/onebit_hybrid.h): the hybrid decoders
+HYBRID_LIB_PATH = os.path.join(_HERE, "csrc", "libonebit_hybrid.so")
+HYBRID_ABI_VERSION = 1
+HYB_BF16, HYB_F32 = 2, 1
+HYBRID_SYMBOLS = {
+    "onebit_hybrid_abi_version": (_int, []),
+    "onebit_hybrid_last_error": (ctypes.c_char_p, []),
+    "onebit_hybrid_workspace_bytes": (ctypes.c_size_t, [_vp, _i64, _i64, ctypes.c_int32, ctypes.c_int32]),
+    "onebit_hybrid_step": (_int, [_vp, _vp, _i64, _i64, ctypes.c_int32, ctypes.c_int32, _vp]),
+    "onebit_hybrid_gemm": (_int, [_vp, _vp, _vp] + [ctypes.c_int32] * 5 + [_vp]),
+    "onebit_hybrid_gemm_splits": (_int, [ctypes.c_int32] * 3),
+}
+
 _lock = threading.Lock()
 _lib = None
+_hybrid = None
 
 
 class OneBitLibraryError(RuntimeError):
     pass
+
+
+def _open(path: str, symbols: dict):
+    try:
+        lib = ctypes.CDLL(path)
+    except OSError as e:  # missing libamdhip64 etc.
+        raise OneBitLibraryError(f"cannot load {path}: {e}") from e
+    for name, (res, args) in symbols.items():
+        try:
+            fn = getattr(lib, name)
+        except AttributeError as e:
+            raise OneBitLibraryError(f"{path} does not export {name}") from e
+        fn.restype, fn.argtypes = res, args
+    return lib
 
 
 def load():
@@ -90,21 +118,34 @@ def load():
             raise OneBitLibraryError(
                 f"{LIB_PATH} not found: build it with `python -m onebit_amd.build` "
                 "(hipcc --offload-arch=gfx950).  There is no CPU fallback.")
-        try:
-            lib = ctypes.CDLL(LIB_PATH)
-        except OSError as e:  # missing libamdhip64 etc.
-            raise OneBitLibraryError(f"cannot load {LIB_PATH}: {e}") from e
-        for name, (res, args) in SYMBOLS.items():
-            try:
-                fn = getattr(lib, name)
-            except AttributeError as e:
-                raise OneBitLibraryError(f"{LIB_PATH} does not export {name}") from e
-            fn.restype, fn.argtypes = res, args
+        lib = _open(LIB_PATH, SYMBOLS)
         v = lib.onebit_abi_version()
         if v != ABI_VERSION:
             raise OneBitLibraryError(f"ABI version mismatch: library {v}, binding {ABI_VERSION}")
         _lib = lib
     return _lib
+
+
+def load_hybrid():
+    """The hybrid decoders' library, loaded and typed once (same rules as ``load``)."""
+    global _hybrid
+    with _lock:
+        if _hybrid is None:
+            if not os.path.exists(HYBRID_LIB_PATH):
+                raise OneBitLibraryError(f"{HYBRID_LIB_PATH} not found: build it with `python -m onebit_amd.build` "
+                                         "(hipcc --offload-arch=gfx950).  There is no CPU fallback.")
+            lib = _open(HYBRID_LIB_PATH, HYBRID_SYMBOLS)
+            v = lib.onebit_hybrid_abi_version()
+            if v != HYBRID_ABI_VERSION:
+                raise OneBitLibraryError(f"ABI version mismatch: library {v}, binding {HYBRID_ABI_VERSION}")
+            _hybrid = lib
+    return _hybrid
+
+
+def check_hybrid(rc: int, what: str):
+    if rc:
+        msg = load_hybrid().onebit_hybrid_last_error().decode("utf-8", "replace")
+        raise ValueError(f"{what}: {msg} (code {rc})") if rc < 0 else RuntimeError(f"{what}: HIP error {rc}: {msg}")
 
 
 def check(rc: int, what: str):

@@ -11,7 +11,9 @@ This module reads and writes exactly that layout and restates the conversion ste
 from __future__ import annotations
 
 import json
+import mmap
 import os
+import struct
 from typing import Dict, Tuple
 
 import torch
@@ -81,3 +83,54 @@ def save_inference_checkpoint(model: OneBitLlamaForCausalLM, path: str) -> Tuple
         json.dump(config_to_json(model.config), f, indent=2)
     torch.save({k: v.detach().cpu() for k, v in model.state_dict().items()}, w_path)
     return cfg_path, w_path
+
+
+_ST_DTYPES = {"F64": torch.float64, "F32": torch.float32, "F16": torch.float16, "BF16": torch.bfloat16, "I64": torch.int64, "I32": torch.int32,
+              "I16": torch.int16, "I8": torch.int8, "U8": torch.uint8, "BOOL": torch.bool}
+
+
+def read_safetensors(path: str) -> Dict[str, torch.Tensor]:
+    """The tensors of a safetensors file: 8-byte little-endian header length, JSON header (name -> dtype, shape, data_offsets), data.
+    Nothing in the file is executed; offsets and sizes are checked.  The tensors are views of a private memory map."""
+    with open(path, "rb") as f:
+        size = os.fstat(f.fileno()).st_size
+        n = struct.unpack("<Q", f.read(8))[0] if size >= 8 else size
+        if n + 8 > size:
+            raise ValueError(f"{path}: truncated header")
+        header = json.loads(f.read(n))
+        buf = mmap.mmap(f.fileno(), 0, access=mmap.ACCESS_COPY)
+    out = {}
+    for name, info in header.items():
+        if name == "__metadata__":
+            continue
+        dt, shape, (a, b) = _ST_DTYPES.get(info["dtype"]), info["shape"], info["data_offsets"]
+        if dt is None:
+            raise ValueError(f"{path}: tensor {name}: dtype {info['dtype']}")
+        count = 1
+        for d in shape:
+            count *= d
+        if a < 0 or b - a != count * torch.empty(0, dtype=dt).element_size() or 8 + n + b > size:
+            raise ValueError(f"{path}: tensor {name}: bytes [{a}, {b}) do not hold {shape} of {info['dtype']}")
+        if count == 0:
+            out[name] = torch.empty(shape, dtype=dt)
+        else:
+            raw = torch.frombuffer(buf, dtype=torch.uint8, count=b - a, offset=8 + n + a)
+            out[name] = (raw if (8 + n + a) % 8 == 0 else raw.clone()).view(dt).view(shape)
+    return out
+
+
+def write_safetensors(path: str, tensors: Dict[str, torch.Tensor]):
+    """``tensors`` as a safetensors file (``read_safetensors`` reads it back)."""
+    names = {v: k for k, v in _ST_DTYPES.items()}
+    header, off = {}, 0
+    for k, t in tensors.items():
+        nb = t.numel() * t.element_size()
+        header[k] = {"dtype": names[t.dtype], "shape": list(t.shape), "data_offsets": [off, off + nb]}
+        off += nb
+    head = json.dumps(header).encode()
+    head += b" " * (-len(head) % 8)
+    with open(path, "wb") as f:
+        f.write(struct.pack("<Q", len(head)))
+        f.write(head)
+        for t in tensors.values():
+            f.write(t.detach().cpu().contiguous().view(-1).view(torch.uint8).numpy().tobytes() if t.numel() else b"")

@@ -1,0 +1,285 @@
+// Dense matrix products of the hybrid decoders (bf16 MFMA with fp32 accumulation; the same kernels in true fp32) for gfx950.
+//
+// FRAGMENT-MAJOR operands: both the weights (packed once at load) and the activations (written that way by their producers) are
+// stored as tiles of 16 rows x KT columns (KT = 32 bf16 / 16 fp32), 1 KB each, in the lane order of the MFMA operand: lane l holds
+// row l & 15, columns (l >> 4) * EPL .. + EPL - 1 (EPL = 8 / 4, 16 bytes).  A tile is one contiguous 1 KB block, so
+//   * a wave streams weights with perfectly linear 1 KB loads (decode: straight from HBM to the operand registers),
+//   * LDS staging is a linear DMA and the operand read a linear ds_read_b128: no swizzle, no bank conflict, no address arithmetic,
+//   * rows and columns are padded to whole tiles at load: the K loop has no masks for any model size.
+// fp32: four v_mfma_f32_16x16x4_f32 per tile pair; element j of every lane's four is one instruction's k, the same on both operands.
+// Products are computed transposed, D[n][t] = sum_k W[n][k] A[t][k]: a lane holds four consecutive output columns n of one token t.
+#pragma once
+#include "ob_common.h"
+
+typedef __bf16 ob_bf8 __attribute__((ext_vector_type(8)));
+typedef __bf16 ob_bf4 __attribute__((ext_vector_type(4)));
+
+template <typename E> struct ObElem;
+template <> struct ObElem<__bf16> {
+    typedef ob_bf8 V16;                       // 16 bytes of operand
+    typedef ob_bf4 V4;
+    static constexpr int EPL = 8, KT = 32;
+    static __device__ __forceinline__ ob_float4 mma(V16 a, V16 b, ob_float4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+};
+template <> struct ObElem<float> {
+    typedef ob_float4 V16;
+    typedef ob_float4 V4;
+    static constexpr int EPL = 4, KT = 16;
+    static __device__ __forceinline__ ob_float4 mma(V16 a, V16 b, ob_float4 c)
+    {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], b[j], c, 0, 0, 0);
+        return c;
+    }
+};
+
+template <typename E> __device__ __forceinline__ typename ObElem<E>::V4 ob_to_v4(ob_float4 v)
+{
+    typename ObElem<E>::V4 o;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o[i] = (E)v[i];
+    return o;
+}
+template <typename E> __device__ __forceinline__ ob_float4 ob_load4f(const E *p)
+{
+    const typename ObElem<E>::V4 v = *reinterpret_cast<const typename ObElem<E>::V4 *>(p);
+    return (ob_float4){(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
+}
+
+// element offset of (row, k) in a fragment-major matrix with nkt tiles per 16-row band
+template <typename E> __host__ __device__ __forceinline__ size_t ob_frag(int row, int k, int nkt)
+{
+    constexpr int EPL = ObElem<E>::EPL, KT = ObElem<E>::KT;
+    return ((size_t)(row >> 4) * nkt + k / KT) * (16 * KT) + (size_t)((k % KT) / EPL) * (16 * EPL) + (row & 15) * EPL + k % EPL;
+}
+
+__device__ __forceinline__ float ob_sigmoidf(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float ob_siluf(float z) { return z * ob_sigmoidf(z); }
+// the 16-bit path's form: exp2 and reciprocal instructions, 1 ulp each in fp32
+__device__ __forceinline__ float ob_silu_fast(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z)); }
+template <typename E> __device__ __forceinline__ float ob_silu(float z)
+{
+    if constexpr (sizeof(E) == 2) return ob_silu_fast(z); else return ob_siluf(z);
+}
+__device__ __forceinline__ float ob_softplusf(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
+
+// ---- what a product's output becomes -------------------------------------------------------------------------------------
+//   OB_EPI_IN     the layer's input product [mixer columns | auxiliary fp32 columns | gate / up tile pairs]:
+//                 mixer columns (+ bias) row-major u[t][n]; auxiliary columns fp32 aux[t][.]; act = silu(gate) * up into the
+//                 fragment-major rows of the output product, at column act_k0
+//   OB_EPI_PART   fp32 partial sums z[split][t][n] (the layer's output product: the row kernel that follows adds the splits)
+//   OB_EPI_LOGITS fp32 logits[t][n], cap * tanh(v / cap) when cap > 0
+enum { OB_EPI_IN = 0, OB_EPI_PART = 1, OB_EPI_LOGITS = 2 };
+
+struct ObDenseArgs {
+    const void *w, *a;             // fragment-major weights [n_tiles][nkt], activations [t tiles][nkt]
+    int n_tiles, nkt, T;
+    int kt_split;                  // k tiles per split (grid.y splits)
+    // OB_EPI_IN
+    const float *bias;             // [16 * nt_mix] or NULL
+    void *u; int nt_mix;           // u: [T][16 * nt_mix]
+    float *aux; int nt_aux;        // aux: [T][16 * nt_aux]; n tile nt_mix + nt_aux opens the gate / up pairs
+    void *act; int act_k0, act_nkt;
+    // OB_EPI_PART
+    float *z; int ldz; size_t z_split;
+    // OB_EPI_LOGITS
+    float *logits; int V; float cap;
+};
+
+// one n-tile pair (nt even) of one token tile: lane = (token t, columns 16 nt + 4 g ..), (token t, columns 16 (nt + 1) + 4 g ..)
+template <typename E, int EPI>
+__device__ __forceinline__ void ob_dense_epilogue(const ObDenseArgs &A, int nt, int t, int g, ob_float4 v0, ob_float4 v1, int split)
+{
+    if (t >= A.T) return;
+    if constexpr (EPI == OB_EPI_PART) {
+        float *z = A.z + (size_t)split * A.z_split + (size_t)t * A.ldz;
+        if (nt < A.n_tiles) *reinterpret_cast<ob_float4 *>(z + nt * 16 + 4 * g) = v0;
+        if (nt + 1 < A.n_tiles) *reinterpret_cast<ob_float4 *>(z + nt * 16 + 16 + 4 * g) = v1;
+    } else if constexpr (EPI == OB_EPI_LOGITS) {
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+            ob_float4 v = h ? v1 : v0;
+            const int n = (nt + h) * 16 + 4 * g;
+            if (A.cap > 0.f) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) v[e] = A.cap * tanhf(v[e] / A.cap);
+            }
+            float *o = A.logits + (size_t)t * A.V + n;
+            if ((A.V & 3) == 0) {
+                if (n < A.V) *reinterpret_cast<ob_float4 *>(o) = v;
+            } else {
+                for (int e = 0; e < 4; ++e) if (n + e < A.V) o[e] = v[e];
+            }
+        }
+    } else {
+        if (nt >= A.n_tiles) return;
+        const int n_plain = A.nt_mix + A.nt_aux;
+        if (nt >= n_plain) {                            // (wave-uniform) gate tile, up tile
+            ob_float4 o;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e] = ob_silu<E>(v0[e]) * v1[e];
+            const int k = A.act_k0 + ((nt - n_plain) >> 1) * 16 + 4 * g;
+            *reinterpret_cast<typename ObElem<E>::V4 *>((E *)A.act + ob_frag<E>(t, k, A.act_nkt)) = ob_to_v4<E>(o);
+            return;
+        }
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+            const int i = nt + h, n = i * 16 + 4 * g;
+            ob_float4 v = h ? v1 : v0;
+            if (i < A.nt_mix) {
+                if (A.bias) v += *reinterpret_cast<const ob_float4 *>(A.bias + n);
+                *reinterpret_cast<typename ObElem<E>::V4 *>((E *)A.u + (size_t)t * (16 * A.nt_mix) + n) = ob_to_v4<E>(v);
+            } else if (i < n_plain) {
+                *reinterpret_cast<ob_float4 *>(A.aux + (size_t)t * (16 * A.nt_aux) + (n - 16 * A.nt_mix)) = v;
+            }
+        }
+    }
+}
+
+// ---- few rows (T <= 64): weights from HBM straight into the operand registers ------------------------------------------
+// Workgroup = 2 n tiles (32 output columns; a gate / up pair) x all token tiles x one K split; its four waves take a quarter of the
+// split's k tiles each and add up through LDS.  Activations come from L2 (1 KB linear loads).  The next U k tiles are requested
+// before the current U are multiplied: U * 2 KB of weights per wave in flight.
+template <typename E, int EPI, int MT>
+__global__ __launch_bounds__(256, MT >= 4 ? 2 : 3) void ob_dense_skinny_kernel(const ObDenseArgs A)
+{
+    typedef typename ObElem<E>::V16 V16;
+    constexpr int U = MT >= 4 ? 2 : 4;
+    __shared__ ob_float4 red[4][2][MT][64];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int nt = blockIdx.x * 2, split = blockIdx.y;
+    const int k_lo = split * A.kt_split, k_hi = min(A.nkt, k_lo + A.kt_split);
+    const int per = (k_hi - k_lo + 3) >> 2;
+    const int k0 = k_lo + wave * per, k1 = min(k0 + per, k_hi);
+    const V16 *w0 = (const V16 *)A.w + (size_t)nt * A.nkt * 64 + lane;
+    const V16 *w1 = (const V16 *)A.w + (size_t)min(nt + 1, A.n_tiles - 1) * A.nkt * 64 + lane;
+    const V16 *ap = (const V16 *)A.a + lane;
+    ob_float4 acc[2][MT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) acc[0][m] = acc[1][m] = (ob_float4){0.f, 0.f, 0.f, 0.f};
+    V16 wc[2][U], ac[MT][U], wn[2][U], an[MT][U];
+    auto fetch = [&](V16 (&wd)[2][U], V16 (&ad)[MT][U], int k) {
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int kk = min(k + u, k1 - 1);
+            wd[0][u] = __builtin_nontemporal_load(w0 + (size_t)kk * 64);
+            wd[1][u] = __builtin_nontemporal_load(w1 + (size_t)kk * 64);
+#pragma unroll
+            for (int m = 0; m < MT; ++m) ad[m][u] = ap[((size_t)m * A.nkt + kk) * 64];
+        }
+    };
+    if (k0 < k1) {                                       // (wave-uniform)
+        fetch(wc, ac, k0);
+        for (int k = k0; k < k1; k += U) {
+            const bool more = k + U < k1;
+            if (more) fetch(wn, an, k + U);
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                if (k + u < k1) {
+#pragma unroll
+                    for (int m = 0; m < MT; ++m) {
+                        acc[0][m] = ObElem<E>::mma(wc[0][u], ac[m][u], acc[0][m]);
+                        acc[1][m] = ObElem<E>::mma(wc[1][u], ac[m][u], acc[1][m]);
+                    }
+                }
+            }
+            if (more) {
+#pragma unroll
+                for (int u = 0; u < U; ++u) {
+                    wc[0][u] = wn[0][u]; wc[1][u] = wn[1][u];
+#pragma unroll
+                    for (int m = 0; m < MT; ++m) ac[m][u] = an[m][u];
+                }
+            }
+        }
+    }
+#pragma unroll
+    for (int h = 0; h < 2; ++h)
+#pragma unroll
+        for (int m = 0; m < MT; ++m) red[wave][h][m][lane] = acc[h][m];
+    __syncthreads();
+    for (int m = wave; m < MT; m += 4) {
+        ob_float4 v[2];
+#pragma unroll
+        for (int h = 0; h < 2; ++h) v[h] = (red[0][h][m][lane] + red[1][h][m][lane]) + (red[2][h][m][lane] + red[3][h][m][lane]);
+        ob_dense_epilogue<E, EPI>(A, nt, m * 16 + (lane & 15), lane >> 4, v[0], v[1], split);
+    }
+}
+
+// ---- many rows: LDS-DMA tiles ------------------------------------------------------------------------------------------
+// Workgroup = NB n tiles x TB token tiles, waves WN x WT; NST stages of one k tile each in LDS, filled by 1 KB DMAs, ONE raw barrier
+// per k tile behind a counted vmcnt: at the top of step k the tile k has landed (at most the NST - 2 younger ones are outstanding),
+// the barrier tells everyone, and the buffer of tile k - 1 -- whose operand reads are complete -- takes tile k + NST - 1.
+__device__ __forceinline__ void ob_dma_1k(const char *base, uint32_t lane_off, uint32_t lds_addr)
+{
+    uint32_t keep;
+    asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %1\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %2, %3\n\ts_mov_b32 m0, %0"
+                 : "=&s"(keep) : "s"(lds_addr), "v"(lane_off), "s"(base) : "memory");
+}
+
+template <typename E, int EPI, int NB, int TB, int WN, int WT, int NST>
+__global__ __launch_bounds__(64 * WN * WT, 2) void ob_dense_tile_kernel(const ObDenseArgs A)
+{
+    typedef typename ObElem<E>::V16 V16;
+    constexpr int NW = WN * WT, TILES = NB + TB, PER = TILES / NW, MN = NB / WN, MT = TB / WT;
+    static_assert(TILES % NW == 0 && NB % WN == 0 && TB % WT == 0 && MN % 2 == 0, "tile shape");
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int wn = wave % WN, wt = wave / WN;
+    // XCD-aware numbering: workgroup ids are dealt round-robin to the 8 XCDs; give each a contiguous range of logical tiles, token
+    // blocks fastest, so that the tiles in flight on an XCD share weight bands and activation rows in its L2
+    const int ntb = (A.T + TB * 16 - 1) / (TB * 16);
+    const int nwg = gridDim.x, orig = blockIdx.x, xcd = orig & 7, q8 = nwg >> 3, rem = nwg & 7;
+    const int bid = (xcd < rem ? xcd * (q8 + 1) : rem * (q8 + 1) + (xcd - rem) * q8) + (orig >> 3);
+    const int nb = bid / ntb, tb = bid - nb * ntb;
+    const int n0 = nb * NB, t0 = tb * TB, split = blockIdx.y;
+    const int k_lo = split * A.kt_split, k_hi = min(A.nkt, k_lo + A.kt_split), nk = k_hi - k_lo;
+    const int t_tiles = (A.T + 15) >> 4;
+    const char *src[PER];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        const int j = wave * PER + i;
+        const size_t band = j < NB ? (size_t)min(n0 + j, A.n_tiles - 1) : (size_t)min(t0 + j - NB, t_tiles - 1);
+        src[i] = (const char *)(j < NB ? A.w : A.a) + (band * A.nkt + k_lo) * 1024;
+    }
+    const uint32_t lds0 = (uint32_t)(size_t)(__attribute__((address_space(3))) char *)smem;
+    const uint32_t lane_off = lane * 16;
+    auto dma = [&](int k, int buf) {
+        const size_t ko = (size_t)min(k, nk - 1) * 1024;
+#pragma unroll
+        for (int i = 0; i < PER; ++i) ob_dma_1k(src[i] + ko, lane_off, lds0 + (uint32_t)(buf * TILES + wave * PER + i) * 1024);
+    };
+    ob_float4 acc[MN][MT];
+#pragma unroll
+    for (int i = 0; i < MN; ++i)
+#pragma unroll
+        for (int j = 0; j < MT; ++j) acc[i][j] = (ob_float4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < NST - 1; ++s) dma(s, s);
+    int buf = 0;
+    for (int k = 0; k < nk; ++k) {
+        asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" :: "n"((NST - 2) * PER) : "memory");
+        dma(k + NST - 1, buf == 0 ? NST - 1 : buf - 1);               // (past the end: the last tile again, into a buffer nobody reads)
+        const V16 *base = reinterpret_cast<const V16 *>(smem + (size_t)buf * TILES * 1024) + lane;
+        V16 wf[MN], af[MT];
+#pragma unroll
+        for (int j = 0; j < MT; ++j) af[j] = base[(NB + wt * MT + j) * 64];
+#pragma unroll
+        for (int i = 0; i < MN; ++i) wf[i] = base[(wn * MN + i) * 64];
+        __builtin_amdgcn_s_setprio(1);
+#pragma unroll
+        for (int i = 0; i < MN; ++i)
+#pragma unroll
+            for (int j = 0; j < MT; ++j) acc[i][j] = ObElem<E>::mma(wf[i], af[j], acc[i][j]);
+        __builtin_amdgcn_s_setprio(0);
+        buf = buf + 1 == NST ? 0 : buf + 1;
+    }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");                  // no transfer may land after the workgroup's LDS is released
+    const int g = lane >> 4;
+#pragma unroll
+    for (int j = 0; j < MT; ++j) {
+        const int t = (t0 + wt * MT + j) * 16 + (lane & 15);
+#pragma unroll
+        for (int i = 0; i < MN; i += 2) ob_dense_epilogue<E, EPI>(A, n0 + wn * MN + i, t, g, acc[i][j], acc[i + 1][j], split);
+    }
+}

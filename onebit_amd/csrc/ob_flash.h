@@ -73,6 +73,37 @@ struct ObFlashRaggedArgs {
     ObFlashSeg seg[OB_FL_MAXSEG];
 };
 
+// How scores become weights.  The kernel below is written once for both:
+//   ObFlSoftmaxF16   fp16 operands, online softmax (the OneBit LLaMA attention)
+//   ObFlSigmoidBf16  bf16 operands, w = 1 / (1 + 2^a), a = q.k (-scale log2 e) + (r1 log2(1 + r2 distance) - pb log2 e), not normalised:
+//                    no maxima, no sums, no rescale.  The distance term of a block depends on query - key only (191 values per
+//                    128 x 64 block): a table in LDS, written beside the block's K / V tiles.  The weights enter the value product as two
+//                    bf16 terms (hi + lo, 16 bits of mantissa): they stay 32-bit quantities up to 2^-17.
+struct ObFlSoftmaxF16 {
+    typedef _Float16 H;
+    typedef ob_half8 V8;
+    static constexpr bool SOFTMAX = true;
+    static __device__ __forceinline__ ob_float4 mfma(V8 a, V8 b, ob_float4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_f16(a, b, c, 0, 0, 0); }
+    typedef ObFlashRaggedArgs RaggedArgs;
+};
+typedef __bf16 ob_fl_bf8 __attribute__((ext_vector_type(8)));
+typedef __bf16 ob_fl_bf4 __attribute__((ext_vector_type(4)));
+typedef __bf16 ob_fl_bf2 __attribute__((ext_vector_type(2)));
+struct ObFlashSigArgs : ObFlashRaggedArgs {      // a.q [rows, H, D], a.k / a.v [slots][Hkv][max_len][D] (bf16); a.scale_log2e NEGATIVE
+    const float *r1, *r2, *pb;                   // [H] each; r1 (with r2) and pb may be NULL
+    void *out; int out_nkt, vdim;                // fragment-major rows of the output product: column head * vdim + d, d < vdim
+};
+struct ObFlSigmoidBf16 {
+    typedef __bf16 H;
+    typedef ob_u32x4 V8;              // (operands kept as dwords: hipcc takes vectors of __bf16 apart and spills)
+    static constexpr bool SOFTMAX = false;
+    static __device__ __forceinline__ ob_float4 mfma(V8 a, V8 b, ob_float4 c)
+    {
+        return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(ob_fl_bf8, a), __builtin_bit_cast(ob_fl_bf8, b), c, 0, 0, 0);
+    }
+    typedef ObFlashSigArgs RaggedArgs;
+};
+
 #define OB_FL_BM 128
 #define OB_FL_BN 64
 #define OB_FL_THREADS 256
@@ -106,9 +137,13 @@ __device__ __forceinline__ float ob_fl_col_sum(float v)
 #define OB_FL_DEFER_THR 8.0f    // log2 units: the running maximum is kept while the new tile's maximum exceeds it by less (P <= 2^8)
 #endif
 
-template <int D, bool RAGGED = false>
-__global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditional_t<RAGGED, ObFlashRaggedArgs, ObFlashArgs> AA)
+template <int D, bool RAGGED = false, class POL = ObFlSoftmaxF16>
+__global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditional_t<RAGGED, typename POL::RaggedArgs, ObFlashArgs> AA)
 {
+    typedef typename POL::H H16;
+    typedef typename POL::V8 V8;
+    constexpr bool SM = POL::SOFTMAX;
+    static_assert(SM || RAGGED, "the sigmoid form has ragged rows only");
     const ObFlashArgs &A = [&]() -> const ObFlashArgs & { if constexpr (RAGGED) return AA.a; else return AA; }();
     constexpr int DT = D / 16, DK = D / 32;
     constexpr int NPC = D / 8;                  // 16-byte pieces per K / V row
@@ -121,8 +156,9 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
     //     r + 1, g - 1 share banks: the 2-way conflicts of rounds 1-3)
     //   V piece pc of row r sits at pc ^ 2 (r mod NPC / 2): the 8 rows a half-wave of the transpose read touches (32 B each)
     //     fall on disjoint banks
-    __shared__ __attribute__((aligned(16))) _Float16 Ks[2][OB_FL_BN][D];
-    __shared__ __attribute__((aligned(16))) _Float16 Vs[2][OB_FL_BN][D];
+    __shared__ __attribute__((aligned(16))) H16 Ks[2][OB_FL_BN][D];
+    __shared__ __attribute__((aligned(16))) H16 Vs[2][OB_FL_BN][D];
+    __shared__ float dist_s[SM ? 1 : 2][SM ? 1 : 192];      // sigmoid: distance term of query - key + 63 of the block
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int lr = lane & 15, g = lane >> 4;
     // XCD-aware numbering: consecutive workgroup ids are dealt round-robin to the 8 XCDs (each with its own 4 MB L2), so
@@ -163,6 +199,12 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
     const __amdgpu_buffer_rsrc_t krs = __builtin_amdgcn_make_buffer_rsrc((void *)(A.k + ((int64_t)b * A.Hkv + kvh) * A.max_len * D), 0, L * D * 2, 0x00020000);
     const __amdgpu_buffer_rsrc_t vrs = __builtin_amdgcn_make_buffer_rsrc((void *)(A.v + ((int64_t)b * A.Hkv + kvh) * A.max_len * D), 0, L * D * 2, 0x00020000);
 
+    float dist_r1 = 0.f, dist_r2 = 0.f, dist_pb = 0.f;
+    if constexpr (!SM) {
+        if (AA.r1) { dist_r1 = AA.r1[head]; dist_r2 = AA.r2[head]; }
+        if (AA.pb) dist_pb = AA.pb[head] * 1.4426950408889634f;
+    }
+
 #ifdef OB_FL_TRACE
     unsigned long long *tr = nullptr;
     if (A.trace && (orig == 0 || orig == nwg / 2) && lane == 0) tr = A.trace + ((orig ? 1 : 0) * (OB_FL_THREADS / 64) + wave) * 66 * 8;
@@ -173,15 +215,15 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
     if (pass == 1 && mb == nmb - 1 - pj) break;                 // odd count: the middle block has no partner
     const int m0 = mb * OB_FL_BM;
     // Q^T fragments of the wave's two query tiles: lane (query = lr, d = 32 ds + 8 g .. + 7)
-    ob_half8 qf[2][DK];
+    V8 qf[2][DK];
     int qpos[2];
 #pragma unroll
     for (int qt = 0; qt < 2; ++qt) {
         const int s = m0 + 32 * wave + 16 * qt + lr;
         qpos[qt] = past + s;                                    // absolute position of this lane's query
-        const _Float16 *qr = A.q + ((qrow0 + min(s, S - 1)) * A.H + head) * D;
+        const H16 *qr = (const H16 *)A.q + ((qrow0 + min(s, S - 1)) * A.H + head) * D;
 #pragma unroll
-        for (int ds = 0; ds < DK; ++ds) qf[qt][ds] = *reinterpret_cast<const ob_half8 *>(qr + 32 * ds + 8 * g);
+        for (int ds = 0; ds < DK; ++ds) qf[qt][ds] = *reinterpret_cast<const V8 *>(qr + 32 * ds + 8 * g);
     }
     ob_float4 acc_o[DT][2];
 #pragma unroll
@@ -217,6 +259,15 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
 #pragma unroll
         for (int j = 0; j < 2 * KLD; ++j) load_piece(kb, j);
     };
+    // sigmoid: distance term of block kb for every query - key of the 128 x 64 block (table entry 63 + query - key)
+    auto dist_table = [&](int buf, int kb) {
+        if constexpr (!SM) {
+            if (tid < 191) {
+                const float d = (float)max(past + m0 - kb * OB_FL_BN + tid - 63, 0);
+                dist_s[buf][tid] = dist_r1 * __builtin_amdgcn_logf(__builtin_fmaf(dist_r2, d, 1.0f)) - dist_pb;
+            }
+        }
+    };
     // operand addresses inside a tile (halves): K row lr of a 16-key tile, piece 4 ds + g; V (transpose read: this lane's chunk of
     // a 4-key x 16-d block = row lr >> 2 of the block, columns 4 (lr & 3) .. + 3; lane group g's block starts at key 4 g)
     typedef short ob_v4s __attribute__((ext_vector_type(4)));
@@ -242,15 +293,15 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
         const int k0 = kb * OB_FL_BN, buf = kb & 1;
         const bool active = !TAIL || k0 <= wave_last_q;     // (wave-uniform) otherwise every key of this block is masked for this wave
         const bool diag = TAIL && (k0 + OB_FL_BN - 1 > past + m0 + 32 * wave || k0 + OB_FL_BN > L);
-        const _Float16 *Kb = &Ks[buf][0][0], *Vb = &Vs[buf][0][0];
+        const H16 *Kb = &Ks[buf][0][0], *Vb = &Vs[buf][0][0];
         const bool do_store = !(OB_FL_ABL & 2) && (!TAIL || kb + 1 < nkb);   // (past the last block the loads returned zeros: harmless)
         const bool do_load = !(OB_FL_ABL & 2) && (!TAIL || kb + 2 < nkb);
         ob_float4 sc[4][2];
         if (active) {
             // ---- S^T = K . Q^T: 4 key tiles x 2 query tiles, K = D.  One staging store rides behind every fourth MFMA.
             // K fragments: 2 DK reads ahead of the MFMAs that consume them (all 4 DK at once would not fit beside the staging registers)
-            ob_half8 kf[4][DK];
-            auto read_k = [&](int i) { kf[i / DK][i % DK] = *reinterpret_cast<const ob_half8 *>(Kb + 16 * (i / DK) * D + koff[i % DK]); };
+            V8 kf[4][DK];
+            auto read_k = [&](int i) { kf[i / DK][i % DK] = *reinterpret_cast<const V8 *>(Kb + 16 * (i / DK) * D + koff[i % DK]); };
 #pragma unroll
             for (int i = 0; i < 2 * DK; ++i) read_k(i);
             __builtin_amdgcn_sched_barrier(0);
@@ -261,32 +312,73 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
 #pragma unroll
             for (int i = 0; i < 4 * DK; ++i) {
 #pragma unroll
-                for (int qt = 0; qt < 2; ++qt) sc[i / DK][qt] = __builtin_amdgcn_mfma_f32_16x16x32_f16(kf[i / DK][i % DK], qf[qt][i % DK], sc[i / DK][qt], 0, 0, 0);
+                for (int qt = 0; qt < 2; ++qt) sc[i / DK][qt] = POL::mfma(kf[i / DK][i % DK], qf[qt][i % DK], sc[i / DK][qt]);
                 __builtin_amdgcn_sched_barrier(0);
                 if (i + 2 * DK < 4 * DK) read_k(i + 2 * DK);
                 __builtin_amdgcn_sched_barrier(0);
             }
-            if (do_store) store_block(buf ^ 1);
+            if (do_store) { store_block(buf ^ 1); dist_table(buf ^ 1, kb + 1); }
             __builtin_amdgcn_sched_barrier(0);
-        } else if (do_store) store_block(buf ^ 1);
+        } else if (do_store) { store_block(buf ^ 1); dist_table(buf ^ 1, kb + 1); }
         OB_FL_T(1);
         if (do_load) load_block(kb + 2);
         OB_FL_T(2);
         if (active) {
-            ob_half8 vf[2][DT];
+            V8 vf[2][DT];
             auto read_v = [&](int ks) {     // A = the 4 keys of key tile 2 ks, then of tile 2 ks + 1, for d = 16 dt + lr (two transpose reads)
 #pragma unroll
                 for (int dt = 0; dt < DT; ++dt) {
                     const ob_v4s lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((ob_lds_v4s *)(Vb + 32 * ks * D + voff[dt]));
                     const ob_v4s hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((ob_lds_v4s *)(Vb + (32 * ks + 16) * D + voff[dt]));
                     const ob_v8s a8 = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
-                    vf[ks][dt] = __builtin_bit_cast(ob_half8, a8);
+                    vf[ks][dt] = __builtin_bit_cast(V8, a8);
                 }
             };
             read_v(0);
             __builtin_amdgcn_sched_barrier(0);
             // ---- causal mask (only blocks that reach this wave's diagonal or the end of the keys), online softmax
-            ob_half8 pb[2][2];
+            V8 pb[2][2];
+            if constexpr (!SM) {
+                // 32 keys at a time: weights of the two key tiles (hi + lo), then their value products -- half the operand registers
+                const float *dt_ = &dist_s[buf][32 * wave + lr + 63 - 4 * g];
+#pragma unroll
+                for (int ks = 0; ks < 2; ++ks) {
+                    ob_u32x4 wh[2], wl[2];
+                    if (ks == 1) {
+                        if (D > 64) __builtin_amdgcn_sched_barrier(0);          // (not before the first half's products: registers)
+                        read_v(1);
+                    }
+#pragma unroll
+                    for (int qt = 0; qt < 2; ++qt) {
+                        if (D > 64) __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+                        for (int i2 = 0; i2 < 4; ++i2) {              // two keys at a time: hi = the weights' upper halves, lo = the rest
+                            float w[2], r[2];
+#pragma unroll
+                            for (int b = 0; b < 2; ++b) {
+                                const int i = 2 * i2 + b, kt = 2 * ks + (i >> 2), e = i & 3;
+                                const float a = __builtin_fmaf(sc[kt][qt][e], A.scale_log2e, dt_[16 * qt - 16 * kt - e]);
+                                w[b] = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(a));
+                                if (TAIL && diag) {
+                                    const int kidx = k0 + 16 * kt + 4 * g + e;
+                                    if (kidx > qpos[qt] || kidx >= L) w[b] = 0.f;
+                                }
+                                r[b] = w[b] - __uint_as_float(__float_as_uint(w[b]) & 0xffff0000u);
+                            }
+                            wh[qt][i2] = __builtin_amdgcn_perm(__float_as_uint(w[1]), __float_as_uint(w[0]), 0x07060302u);
+                            wl[qt][i2] = __builtin_bit_cast(uint32_t, __builtin_convertvector((ob_float2){r[0], r[1]}, ob_fl_bf2));
+                        }
+                    }
+                    if (D > 64) __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+                    for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+                        for (int qt = 0; qt < 2; ++qt) {
+                            acc_o[dt][qt] = POL::mfma(vf[ks][dt], __builtin_bit_cast(V8, wh[qt]), acc_o[dt][qt]);
+                            acc_o[dt][qt] = POL::mfma(vf[ks][dt], __builtin_bit_cast(V8, wl[qt]), acc_o[dt][qt]);
+                        }
+                }
+            } else {
 #if OB_FL_ABL & 1
 #pragma unroll
             for (int qt = 0; qt < 2; ++qt)
@@ -359,7 +451,8 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
 #pragma unroll
                 for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
-                    for (int qt = 0; qt < 2; ++qt) acc_o[dt][qt] = __builtin_amdgcn_mfma_f32_16x16x32_f16(vf[ks][dt], pb[qt][ks], acc_o[dt][qt], 0, 0, 0);
+                    for (int qt = 0; qt < 2; ++qt) acc_o[dt][qt] = POL::mfma(vf[ks][dt], pb[qt][ks], acc_o[dt][qt]);
+            }
         }
         OB_FL_T(4);
         __syncthreads();                        // block kb + 1 is complete in the other buffer; this one may be overwritten
@@ -367,6 +460,7 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
     const int nfull = min((past + m0 + 1) / OB_FL_BN, nkb);     // blocks entirely below every wave's diagonal
     load_block(0);
     store_block(0);
+    dist_table(0, 0);
     load_block(1);
     __syncthreads();
     OB_FL_TP(1);
@@ -379,6 +473,28 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
 #pragma unroll
     for (int qt = 0; qt < 2; ++qt) {
         const int s = m0 + 32 * wave + 16 * qt + lr;
+        if constexpr (!SM) {
+            if (s >= S) continue;
+            const int row = (int)qrow0 + s;
+            H16 *o = (H16 *)AA.out + ((size_t)(row >> 4) * AA.out_nkt) * 512 + (row & 15) * 8;          // fragment-major row `row`
+#pragma unroll
+            for (int dt = 0; dt < DT; ++dt) {
+                const int d = 16 * dt + 4 * g, c = head * AA.vdim + d;
+                if ((AA.vdim & 3) == 0) {
+                    if (d < AA.vdim) {
+                        ob_fl_bf4 ov;
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) ov[e] = (H16)acc_o[dt][qt][e];
+                        *reinterpret_cast<ob_fl_bf4 *>(o + (c >> 5) * 512 + ((c & 31) >> 3) * 128 + (c & 7)) = ov;
+                    }
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e)
+                        if (d + e < AA.vdim) o[((c + e) >> 5) * 512 + (((c + e) & 31) >> 3) * 128 + ((c + e) & 7)] = (H16)acc_o[dt][qt][e];
+                }
+            }
+            continue;
+        } else {
         const float l = ob_fl_col_sum(l_run[qt]);
         const float inv = l > 0.f ? 1.0f / l : 0.f;
         if (s >= S) continue;
@@ -390,6 +506,7 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
             for (int e = 0; e < 4; ++e) ov[e] = (_Float16)(acc_o[dt][qt][e] * inv);
             if (A.h_next) ov = ov * *reinterpret_cast<const ob_half4 *>(A.h_next + head * D + 16 * dt + 4 * g);
             *reinterpret_cast<ob_half4 *>(orow + 16 * dt + 4 * g) = ov;
+        }
         }
     }
     OB_FL_TP(3);

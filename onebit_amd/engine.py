@@ -554,6 +554,80 @@ class BatchedDecodeStep:
         return self.buf["x"]
 
 
+class StagedItems:
+    """One scheduler step as the row arrays its kernels read (device addresses) plus the host-side segment list."""
+    __slots__ = ("n_rows", "n_dec", "n_out", "dec_ctx", "segs", "tokens", "row_slot", "row_pos", "row_off", "out_rows")
+
+
+class ItemStage:
+    """Turns ``(slot, start, tokens[, out])`` items into row arrays on the device: single-token items first, then the prompt chunks, each
+    row with its slot, position and offset inside its item.  ``out``: how many of the item's last rows are sampled (default 1), or the
+    list of its rows (offsets, ascending) that are.  One pinned staging row and ONE asynchronous copy per step; two of them in turn, each guarded by an
+    event, so that a caller who enqueues steps without synchronising never rewrites a row in flight."""
+
+    def __init__(self, device, n_slots: int, max_len: int, vocab: int):
+        self.dev, self.n_slots, self.max_len, self.vocab = device, int(n_slots), int(max_len), int(vocab)
+        self.rows, self._turn = 0, 0
+
+    def ensure(self, rows: int):
+        if rows <= self.rows:
+            return
+        n = 5 * rows + self.n_slots
+        self._h = [torch.zeros(n, dtype=torch.int32).pin_memory() for _ in range(2)]
+        self._np = [h.numpy() for h in self._h]
+        self._ev = [None, None]
+        self._d = [torch.zeros(n, dtype=torch.int32, device=self.dev) for _ in range(2)]
+        self.rows = rows
+
+    def stage(self, items) -> StagedItems:
+        n_items = len(items)
+        if n_items == 0 or n_items > self.n_slots:
+            raise ValueError(f"step: {n_items} items for {self.n_slots} slots")
+        R, V = self.rows, self.vocab
+        sb, self._turn = self._turn, self._turn ^ 1
+        if self._ev[sb] is not None:
+            self._ev[sb].synchronize()
+        st = self._np[sb]
+        tok, rs, rp, ro, outr = st[:R], st[R:2 * R], st[2 * R:3 * R], st[3 * R:4 * R], st[4 * R:]
+        order = sorted(range(n_items), key=lambda i: len(items[i][2]) != 1)          # single-token rows first (stable)
+        outs = [it[3] if len(it) > 3 else 1 for it in items]
+        outs = [list(o) if isinstance(o, (list, tuple)) else list(range(len(it[2]) - int(o), len(it[2]))) for o, it in zip(outs, items)]
+        out0, n_out = [], 0
+        for o in outs:
+            out0.append(n_out)
+            n_out += len(o)
+        s = StagedItems()
+        s.segs, row, s.n_dec, s.dec_ctx, seen = [], 0, 0, 0, set()
+        for i in order:
+            slot, start, toks = items[i][:3]
+            n = len(toks)
+            if any(not 0 <= o < n for o in outs[i]) or (len(items[i]) > 3 and not isinstance(items[i][3], (list, tuple)) and not outs[i]):
+                raise ValueError(f"step: item {i} asks for output rows {outs[i]} of {n}")
+            if n < 1 or not 0 <= slot < self.n_slots or start < 0 or start + n > self.max_len or slot in seen:
+                raise ValueError(f"step: item {i} (slot {slot}, start {start}, {n} tokens) outside the cache or a repeated slot")
+            if min(toks) < 0 or max(toks) >= V:
+                raise ValueError(f"step: item {i} has a token outside the vocabulary")
+            seen.add(slot)
+            tok[row:row + n] = toks
+            rs[row:row + n] = slot
+            rp[row:row + n] = range(start, start + n)
+            ro[row:row + n] = range(n)
+            if n == 1:
+                s.n_dec += 1
+                s.dec_ctx = max(s.dec_ctx, start + 1)
+            else:
+                s.segs.append((row, n, slot, start))
+            outr[out0[i]:out0[i] + len(outs[i])] = [row + o for o in outs[i]]
+            row += n
+        self._d[sb].copy_(self._h[sb], non_blocking=True)                            # stream-ordered before the kernels
+        self._ev[sb] = torch.cuda.Event()
+        self._ev[sb].record(torch.cuda.current_stream(self.dev))
+        base = self._d[sb].data_ptr()
+        s.n_rows, s.n_out = row, n_out
+        s.tokens, s.row_slot, s.row_pos, s.row_off, s.out_rows = (base + 4 * k * R for k in range(5))
+        return s
+
+
 class MixedStep:
     """``onebit_mixed_step`` bound to a model and its KV-cache slots: ONE scheduler step of continuous batching
     on native kernels -- the token rows of all scheduled items concatenated, every 1-bit projection one GEMM over all rows, fused
@@ -593,6 +667,7 @@ class MixedStep:
         self.lib.onebit_mixed_workspace_bytes.argtypes = [ctypes.POINTER(_Model), _i64, _i32, _i32]
         self.lib.onebit_mixed_step.argtypes = [ctypes.POINTER(_Model), ctypes.POINTER(_MixedState), _vp]
         self._rows = 0
+        self._stage = ItemStage(dev, self.n_slots, self.max_len, cfg.vocab_size)
         self._ensure(int(max_rows))
         self.launches = 0
 
@@ -606,12 +681,7 @@ class MixedStep:
         self._ws = None                                           # (free the old block first)
         self._ws = torch.zeros(nb + 256, dtype=torch.uint8, device=dev)
         self._ws_off = (-self._ws.data_ptr()) % 256
-        # one pinned staging row [tokens | row_slot | row_pos | out_rows] and ONE asynchronous copy per step; two of them in turn,
-        # each guarded by an event, so that a caller who enqueues steps without synchronising never rewrites a row in flight
-        self._h_stage = [torch.zeros(4 * rows + ns, dtype=torch.int32).pin_memory() for _ in range(2)]
-        self._h_np = [h.numpy() for h in self._h_stage]
-        self._h_ev = [None, None]
-        self._d_stage = [torch.zeros(4 * rows + ns, dtype=torch.int32, device=dev) for _ in range(2)]
+        self._stage.ensure(rows)
         self.next_tokens = torch.zeros(rows + ns, dtype=torch.int32, device=dev)
         self._rows = rows
         self._ensure_logits(ns)
@@ -628,58 +698,17 @@ class MixedStep:
         one per item in the order given (the token after the item's LAST row: for a prompt chunk that is not the prompt's last one
         the caller ignores it).  An item may carry a fourth element ``k`` (default 1): lm_head runs on its last ``k`` rows (the
         evaluation caller scores a request's continuation rows) and the item contributes ``k`` consecutive entries to the returned
-        tokens and to ``logits``.  Asynchronous: synchronise before reading."""
-        n_items = len(items)
-        if n_items == 0 or n_items > self.n_slots:
-            raise ValueError(f"MixedStep.launch: {n_items} items for {self.n_slots} slots")
-        T = sum(len(it[2]) for it in items)
-        self._ensure(T)
-        R, ns, V = self._rows, self.n_slots, self.cfg.vocab_size
-        sb = self.launches & 1
-        if self._h_ev[sb] is not None:
-            self._h_ev[sb].synchronize()
-        st = self._h_np[sb]
-        tok, rs, rp, outr = st[:R], st[R:2 * R], st[2 * R:3 * R], st[3 * R:]
-        order = sorted(range(n_items), key=lambda i: len(items[i][2]) != 1)          # single-token rows first (stable)
-        outs = [int(it[3]) if len(it) > 3 else 1 for it in items]
-        out0 = [0] * n_items
-        for i in range(1, n_items):
-            out0[i] = out0[i - 1] + outs[i - 1]
-        n_out = out0[-1] + outs[-1]
-        self._ensure_logits(n_out)
-        segs, row, n_dec, dec_ctx, seen = [], 0, 0, 0, set()
-        for i in order:
-            slot, start, toks = items[i][:3]
-            n = len(toks)
-            if not 1 <= outs[i] <= n:
-                raise ValueError(f"MixedStep.launch: item {i} asks for {outs[i]} output rows of {n}")
-            if n < 1 or not 0 <= slot < ns or start < 0 or start + n > self.max_len or slot in seen:
-                raise ValueError(f"MixedStep.launch: item {i} (slot {slot}, start {start}, {n} tokens) outside the cache or a repeated slot")
-            if min(toks) < 0 or max(toks) >= V:
-                raise ValueError(f"MixedStep.launch: item {i} has a token outside the vocabulary")
-            seen.add(slot)
-            tok[row:row + n] = toks
-            rs[row:row + n] = slot
-            rp[row:row + n] = range(start, start + n)
-            if n == 1:
-                n_dec += 1
-                dec_ctx = max(dec_ctx, start + 1)
-            else:
-                segs.append((row, n, slot, start))
-            outr[out0[i]:out0[i] + outs[i]] = range(row + n - outs[i], row + n)
-            row += n
-        d = self._d_stage[sb]
-        d.copy_(self._h_stage[sb], non_blocking=True)                                # stream-ordered before the kernels
-        self._h_ev[sb] = torch.cuda.Event()
-        self._h_ev[sb].record(torch.cuda.current_stream(self.dev))
-        seg_arr = (_Seg * max(len(segs), 1))(*[_Seg(*g) for g in segs])
-        base = d.data_ptr()
-        state = _MixedState(ctypes.sizeof(_MixedState), T, n_dec, len(segs), n_out, ns, self.attn_chunk, dec_ctx,
-                            base, base + 4 * R, base + 8 * R, seg_arr, base + 12 * R, self.next_tokens.data_ptr(),
+        tokens and to ``logits``; or the list of the item's rows that lm_head runs on.  Asynchronous: synchronise before reading."""
+        self._ensure(sum(len(it[2]) for it in items))
+        self._ensure_logits(sum((len(it[3]) if isinstance(it[3], (list, tuple)) else int(it[3])) if len(it) > 3 else 1 for it in items))
+        g = self._stage.stage(items)
+        seg_arr = (_Seg * max(len(g.segs), 1))(*[_Seg(*x) for x in g.segs])
+        state = _MixedState(ctypes.sizeof(_MixedState), g.n_rows, g.n_dec, len(g.segs), g.n_out, self.n_slots, self.attn_chunk, g.dec_ctx,
+                            g.tokens, g.row_slot, g.row_pos, seg_arr, g.out_rows, self.next_tokens.data_ptr(),
                             None if self.logits is None else self.logits.data_ptr(), self._part_val.data_ptr(), self._part_idx.data_ptr(),
                             self._ws.data_ptr() + self._ws_off, self._ws.numel() - self._ws_off)
         with torch.cuda.device(self.dev):
             rc = self.lib.onebit_mixed_step(ctypes.byref(self._model), ctypes.byref(state), torch.cuda.current_stream(self.dev).cuda_stream)
         _lib.check(rc, "onebit_mixed_step")
         self.launches += 1
-        return self.next_tokens[:n_out]
+        return self.next_tokens[:g.n_out]

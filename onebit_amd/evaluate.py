@@ -86,6 +86,8 @@ def _ragged_scorer(model, n_slots: int, max_len: int, any_dtype: bool = False):
     """A ``MixedStep`` over ``n_slots`` fresh KV-cache slots for the ragged route of ``loglikelihood_tokens``; None when the
     native step does not take the model (CPU, another model class, head_dim other than 64 / 128)."""
     try:
+        if hasattr(model, "step_engine"):                       # a family with its own step engine (fp32 logits whatever its operands)
+            return model.step_engine(n_slots, max_len, max_rows=64)
         from .engine import MixedStep, fp16_view
         from .llama import KVCache, OneBitLlamaForCausalLM
         if not isinstance(model, OneBitLlamaForCausalLM) or not model.lm_head.weight.is_cuda:

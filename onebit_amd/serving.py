@@ -54,6 +54,27 @@ class Item:                           # one request's share of a step
     start: int                        # position of tokens[0]
 
 
+class SlotPool:
+    """The free slots of a cache or state manager, lowest number first."""
+
+    def __init__(self, n: int):
+        self.n = n
+        self._free = list(range(n - 1, -1, -1))
+
+    def __len__(self) -> int:
+        return len(self._free)
+
+    def take(self) -> int:
+        return self._free.pop()
+
+    def give(self, slot: int):
+        self._free.append(slot)
+
+    def grow(self, n: int):
+        self._free = list(range(n - 1, self.n - 1, -1)) + self._free
+        self.n = n
+
+
 class Scheduler:
     """FIFO admission into ``max_batch`` KV-cache slots; a step schedules the whole prompt of every
     newly admitted request (bounded by ``max_step_tokens``) plus one token per running request.
@@ -83,7 +104,7 @@ class Scheduler:
         self.waiting: Deque[Request] = deque()
         self.running: List[Request] = []
         self.finished: Dict[int, Request] = {}
-        self._free = list(range(max_batch - 1, -1, -1))
+        self._free = SlotPool(max_batch)
         self._next = 0
 
     def add(self, prompt: List[int], max_new_tokens: int) -> int:
@@ -142,7 +163,7 @@ class Scheduler:
             if n == 0:
                 break                                                         # FIFO: no overtaking
             self.waiting.popleft()
-            r.slot = self._free.pop()
+            r.slot = self._free.take()
             self.running.append(r)
             items.append(Item(r, r.prompt[:n], 0))
             if budget is not None:
@@ -166,7 +187,7 @@ class Scheduler:
                 done.append(r)
         for r in done:
             self.running.remove(r)
-            self._free.append(r.slot)
+            self._free.give(r.slot)
             self.finished[r.rid] = r
         return done
 
@@ -179,6 +200,18 @@ class ContinuousBatcher:
         (``onebit_decode_step_batched`` with ``attn_splits``: ``attn_chunk`` positions per workgroup, one graph per power-of-two
         split count) instead of the one-workgroup-per-(head, slot) form -- measured at 32 slots on 7B: equal at 128 cached
         tokens (2.37 ms), 2.64 vs 2.81 ms at 256, 3.23 vs 3.61 at 512 (tools/serve_ctx_probe.py), and the only form once 4 * max_len + 5.4 KB of scores no longer fit the LDS."""
+        self.steps = 0
+        self.tokens_scheduled = 0
+        self.graph_steps = self.mixed_steps = self.long_steps = 0
+        self.time_mixed = self.time_decode = 0.0     # wall seconds in steps with / without prompt tokens (each step ends in a host sync)
+        self._engine = None
+        if hasattr(model, "step_engine"):
+            # a family that brings its own step engine and state manager (onebit_amd/hybrid.py): every step, mixed or decode-only, is one
+            # launch of it on this scheduler's items
+            self.model = model
+            self.sched = Scheduler(max_batch, max_len, max_step_tokens, prefill_chunk)
+            self._engine = model.step_engine(max_batch, max_len, max_rows=max_step_tokens or 256, use_graph=use_graph)
+            return
         p = model.lm_head.weight
         if not p.is_cuda:
             raise RuntimeError("ContinuousBatcher needs the model on a ROCm GPU (no CPU fallback)")
@@ -192,8 +225,6 @@ class ContinuousBatcher:
         self.cache = [(torch.zeros(shape, device=self.dev, dtype=self.dtype),
                        torch.zeros(shape, device=self.dev, dtype=self.dtype)) for _ in range(cfg.num_hidden_layers)]
         self.cos, self.sin = model._rope_tables(self.dev, self.dtype)
-        self.steps = 0
-        self.tokens_scheduled = 0
         # decode-only steps (the steady state) run as ONE HIP graph over static shapes: row i = slot i,
         # idle slots compute on token 0 at position 0 of their own (unused) cache slot
         self.use_graph = use_graph
@@ -218,13 +249,11 @@ class ContinuousBatcher:
         self._graph_fb = None
         self._g_ring = torch.zeros(self.max_burst, max_batch, dtype=torch.long, device=self.dev)
         self._h_ring = torch.zeros(self.max_burst, max_batch, dtype=torch.long).pin_memory()
-        self.graph_steps = 0
         # native batched step (onebit_decode_step_batched) for the decode-only graph; torch-op glue otherwise
         self._native = None
         self._long = {}                         # split count -> (BatchedDecodeStep with attn_splits, its HIP graph)
         self.long_context_from, self.attn_chunk = int(long_context_from), int(attn_chunk)
         self._short_ok = 512 + 3 * 128 * 2 + 8 * 128 * 4 + 4 * max_len <= 64 * 1024       # the one-workgroup form's LDS bound
-        self.long_steps = 0
         if native and use_graph and 2 <= max_batch <= 64 and self.dtype == torch.float16 and cfg.head_dim <= 128:
             from .engine import BatchedDecodeStep
             try:
@@ -239,8 +268,6 @@ class ContinuousBatcher:
         # lm_head on the sampling rows); `_forward` below (torch glue in the reference's op order) remains for native=False and
         # for checkpoints the native step refuses (head_dim other than 64 / 128, in_features % 32 != 0, fp32 parameters)
         self._mixed = None
-        self.mixed_steps = 0
-        self.time_mixed = self.time_decode = 0.0     # wall seconds in steps with / without prompt tokens (each step ends in a host sync)
         if native and self.dtype == torch.float16:
             from .engine import MixedStep
             try:
@@ -495,6 +522,14 @@ class ContinuousBatcher:
                 self.time_mixed += time.perf_counter() - t0
 
     def _run_items(self, items: List[Item]) -> List[Request]:
+        if self._engine is not None:
+            graphs = self._engine.graph_launches
+            nxt = self._engine.step([(it.req.slot, it.start, it.tokens) for it in items])
+            if self._engine.graph_launches > graphs:
+                self.graph_steps += 1
+            else:
+                self.mixed_steps += 1
+            return self.sched.commit(items, nxt)
         if self.use_graph and all(len(it.tokens) == 1 for it in items):
             n = self._burst_len(items)
             if n <= 1:
@@ -521,3 +556,56 @@ class ContinuousBatcher:
             if after == before:            # an empty plan with work pending would spin forever
                 raise RuntimeError("ContinuousBatcher.run: no progress (a waiting prompt exceeds the step budget?)")
         return {rid: r.out for rid, r in self.sched.finished.items()}
+
+
+def eos_set(eos_token_id, pad_token_id, batch: int):
+    """(set of EOS ids or None, pad id) with ``generate``'s rules: EOS with more than one row needs a pad id (generation/utils.py:2543)."""
+    if eos_token_id is None:
+        return None, pad_token_id
+    eos = set(eos_token_id) if isinstance(eos_token_id, (list, tuple, set)) else {int(eos_token_id)}
+    if pad_token_id is None:
+        if batch > 1:
+            raise ValueError("generate: eos_token_id with batch > 1 needs pad_token_id (generation/utils.py:2543)")
+        pad_token_id = next(iter(eos)) if not isinstance(eos_token_id, (list, tuple)) else int(eos_token_id[0])
+    return eos, pad_token_id
+
+
+def cut_at_eos(rows: List[List[int]], eos, pad_token_id) -> List[List[int]]:
+    """EOS applied to rows generated without looking: a finished row continues with the pad id, the output ends where every row is
+    finished (generation/utils.py:2543-2570)."""
+    if eos is None:
+        return rows
+    ends = [next((j + 1 for j, t in enumerate(r) if t in eos), len(r)) for r in rows]
+    n = max(ends)
+    return [r[:e] + [pad_token_id] * (n - e) for r, e in zip(rows, ends)]
+
+
+def batched_rows(model, prompts: List[List[int]], max_new_tokens: int, max_positions: int, engines: Dict) -> List[List[int]]:
+    """Greedy tokens of every prompt through a ``ContinuousBatcher`` with one slot per row, kept per (rows, length bucket) in ``engines``."""
+    max_len = max(len(p) for p in prompts) + max_new_tokens
+    if max_len > max_positions:
+        raise ValueError("prompt + max_new_tokens exceeds max_position_embeddings")
+    key = (len(prompts), min(-(-max_len // 256) * 256, max_positions))
+    cb = engines.get(key)
+    if cb is None:
+        if len(engines) >= 4:
+            engines.clear()
+        cb = engines[key] = ContinuousBatcher(model, max_batch=key[0], max_len=key[1])
+    ids = [cb.add_request(p, max_new_tokens) for p in prompts]
+    out = cb.run()
+    rows = [out[i] for i in ids]
+    for i in ids:
+        cb.sched.finished.pop(i, None)
+    return rows
+
+
+@torch.no_grad()
+def generate_batched(model, input_ids: torch.Tensor, max_new_tokens: int, eos_token_id=None, pad_token_id=None, engines: Optional[Dict] = None) -> torch.Tensor:
+    """``generate``'s contract (input_ids [B, S] -> prompts followed by up to ``max_new_tokens`` greedy tokens) on the batcher."""
+    if input_ids.dim() != 2:
+        raise ValueError("input_ids must be [B, S]")
+    if max_new_tokens < 1:
+        return input_ids
+    eos, pad = eos_set(eos_token_id, pad_token_id, input_ids.shape[0])
+    rows = cut_at_eos(batched_rows(model, input_ids.tolist(), max_new_tokens, model.max_positions, {} if engines is None else engines), eos, pad)
+    return torch.cat([input_ids.to(model.device), torch.tensor(rows, dtype=input_ids.dtype, device=model.device)], dim=1)

@@ -1,0 +1,81 @@
+"""Replay a trace: given token ids through a model step by step, logits out.  Nothing is sampled; the steps run on the family's step
+engine over its cache / state slots, as the batcher's do.
+
+Standard input, one JSON object a line:
+  {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
+``entries``: each request's next tokens and the places among them whose logits are wanted; ``end``: requests finished after the step (their
+slots are given back).  A step in which something is wanted writes OUT/<step>.f32, little-endian fp32 [wanted, vocab] in entry order;
+after every step ``done <step>`` is printed."""
+from __future__ import annotations
+
+import json
+import os
+import sys
+from typing import Dict, List, Optional, Tuple
+
+import torch
+
+from .registry import find_family, load_model
+from .serving import SlotPool
+
+
+class TraceSession:
+    """Requests by name on the slots of a step engine: which slot each holds and how many tokens it has."""
+
+    def __init__(self, family, model, max_len: int, n_slots: int = 8):
+        self.engine = family.engine(model, n_slots, max_len)
+        self.pool = SlotPool(n_slots)
+        self.live: Dict[str, Tuple[int, int]] = {}
+
+    def step(self, entries: List[dict], end: List[str] = ()) -> Optional[torch.Tensor]:
+        """One step of ``entries`` as one batch; fp32 logits [wanted, vocab] on the host, or None."""
+        entries = [e for e in entries if e["tokens"]]
+        new = sum(e["id"] not in self.live for e in entries)
+        if new > len(self.pool):
+            n = max(2 * self.pool.n, self.pool.n + new - len(self.pool))
+            self.engine.grow(n)
+            self.pool.grow(n)
+        items = []
+        for e in entries:
+            slot, pos = self.live[e["id"]] if e["id"] in self.live else (self.pool.take(), 0)
+            items.append((slot, pos, list(e["tokens"]), list(e["want"])))
+            self.live[e["id"]] = (slot, pos + len(e["tokens"]))
+        wanted = sum(len(it[3]) for it in items)
+        out = None
+        if items:
+            # a step of single tokens samples every row anyway (one graph); the rows that are wanted are picked below
+            single = all(len(it[2]) == 1 for it in items)
+            self.engine.launch([it[:3] for it in items] if single else items)
+            if wanted:
+                rows = [i for i, it in enumerate(items) for _ in it[3]] if single else list(range(wanted))
+                out = self.engine.logits[rows].float().cpu()
+            elif torch.cuda.is_available():
+                torch.cuda.synchronize()
+        for rid in end:
+            if rid in self.live:
+                self.pool.give(self.live.pop(rid)[0])
+        return out
+
+
+def run(model_dir: str, dtype: str, out_dir: str, max_tokens: int, device: str = "cuda", lines=None, stdout=None) -> int:
+    """The trace runner's main loop; returns the exit code (3: the family's kernels do not run in fp32)."""
+    fam = find_family(model_dir)
+    if dtype == "float32" and not fam.float32:
+        print(f"{fam.name}: the step kernels do not run in float32", file=sys.stderr)
+        return 3
+    model = load_model(model_dir, device, torch.float32 if dtype == "float32" else None)
+    session = TraceSession(fam, model, max(1, min(max_tokens, fam.max_positions(model))))
+    os.makedirs(out_dir, exist_ok=True)
+    stdout = stdout or sys.stdout
+    for line in lines if lines is not None else sys.stdin:
+        if not line.strip():
+            continue
+        st = json.loads(line)
+        logits = session.step(st["entries"], st.get("end") or [])
+        if logits is not None:
+            part = os.path.join(out_dir, f".{st['step']}.part")
+            with open(part, "wb") as f:
+                f.write(logits.contiguous().numpy().astype("<f4").tobytes())
+            os.replace(part, os.path.join(out_dir, f"{st['step']}.f32"))
+        print(f"done {st['step']}", file=stdout, flush=True)
+    return 0
