@@ -65,6 +65,101 @@ def spawn_command(gpus, argv, port=None):
             "--master-addr", "127.0.0.1", "--master-port", str(port), os.path.abspath(__file__)] + list(argv)
 
 
+# --hybrid: width -> (feed-forward, attention heads x head size, state-space heads x head size, state, groups): layers of the proportions of
+# real models; four state-space + four attention layers, random weights
+HYBRID_SIZES = {1024: (2816, 16, 64, 32, 64, 64, 1), 2048: (5632, 16, 128, 64, 64, 128, 1), 4096: (11008, 32, 128, 128, 64, 128, 8)}
+
+
+def hybrid_config(width, layers=8, vocab=32000, max_positions=4096):
+    from onebit_amd.lebepel import LebepelConfig
+    ff, ah, ad, sh, sd, n, g = HYBRID_SIZES[width]
+    mlp = {"kind": "dense", "ff": ff}
+    ssm = {"type": "mamba2", "mixer": {"heads": sh, "groups": g, "state": n, "vdim": sd, "conv": 4, "norm_groups": g}, "mlp": mlp}
+    att = {"type": "attention", "mixer": {"heads": ah, "kv_heads": ah, "dim": ad, "vdim": ad, "scale": ad ** -0.5}, "mlp": mlp}
+    return LebepelConfig(vocab_size=vocab, width=width, layers=[ssm, att] * (layers // 2), norm_eps=1e-5, residual_mult=0.5, logit_softcap=30.0,
+                         max_positions=max_positions)
+
+
+def measure_hybrid(dev, what="all", widths=(2048, 4096), beside=True, layers=8):
+    """Prefill and decode throughput of the hybrid decoder at a few sizes, and of the 1-bit LLaMA with the same width, feed-forward, heads and
+    number of layers: prompts through the step engines (``HybridStep`` / ``MixedStep``), decoding by their graphs."""
+    from onebit_amd.engine import MixedStep
+    from onebit_amd.lebepel import build_synthetic_model
+    from onebit_amd.llama import OneBitLlamaConfig, KVCache
+    from onebit_amd.llama import build_synthetic_model as build_onebit
+    from onebit_amd.serving import ContinuousBatcher, Item, Request
+    g = torch.Generator().manual_seed(0)
+    prompts = [(1, 512), (1, 2048), (8, 2048)]
+    decodes = [(1, 512), (32, 512), (32, 2000)]
+
+    def clock(fn, iters):
+        fn(); fn()
+        torch.cuda.synchronize(dev)
+        ts = []
+        for _ in range(3):
+            t0 = time.perf_counter()
+            for _ in range(iters):
+                fn()
+            torch.cuda.synchronize(dev)
+            ts.append((time.perf_counter() - t0) / iters)
+        return sorted(ts)[1]
+
+    out = []
+    for width in widths:
+        ff, ah, ad = HYBRID_SIZES[width][:3]
+        row = {"width": width, "ff": ff, "layers": layers}
+        for name in ("lebepel", "onebit_llama") if beside else ("lebepel",):
+            if name == "lebepel":
+                cfg = hybrid_config(width, layers)
+                model = build_synthetic_model(cfg, 1, torch.bfloat16, dev)
+                per_layer = [sum(a * b for a, b in (s for k, s in cfg.tensor_shapes().items() if k.startswith("l%d." % i) and len(s) == 2 and "conv" not in k))
+                             for i in range(2)]
+                flops_row = layers // 2 * sum(per_layer) * 2
+            else:
+                cfg = OneBitLlamaConfig(vocab_size=32000, hidden_size=width, intermediate_size=ff, num_hidden_layers=layers, num_attention_heads=ah,
+                                        max_position_embeddings=4096)
+                model = build_onebit(cfg, 1, device=dev)
+                flops_row = layers * (4 * width * width + 3 * width * ff) * 2
+            r = row[name] = {"linear_GFLOP_per_token": round(flops_row / 1e9, 3), "prefill": [], "decode": []}
+            if what in ("all", "prefill"):
+                for B, S in prompts:
+                    toks = [torch.randint(0, 32000, (S,), generator=g).tolist() for _ in range(B)]
+                    if name == "lebepel":
+                        eng = model.step_engine(B, S, max_rows=B * S)
+                    else:
+                        eng = MixedStep(model, KVCache(cfg, B, S, dev, torch.float16).layers, B, S, max_rows=B * S)
+                    t = clock(lambda: eng.launch([(b, 0, toks[b]) for b in range(B)]), 5)
+                    r["prefill"].append({"batch": B, "prompt": S, "ms": round(t * 1e3, 3), "tokens_per_s": round(B * S / t), "linear_TFLOPs": round(B * S * flops_row / t / 1e12, 1)})
+                    del eng
+                    torch.cuda.empty_cache()
+            if what in ("all", "decode"):
+                for B, ctx in decodes:
+                    # steps at a fixed context, enqueued back to back: the engine's graph replay, state and cache holding whatever they hold
+                    n_it = 40
+                    if name == "lebepel":
+                        eng = model.step_engine(B, ctx + 8)
+                        t = clock(lambda: eng.launch([(b, ctx, [b + 1]) for b in range(B)]), n_it)
+                    elif B == 1:
+                        from onebit_amd.engine import DecodeEngine
+                        eng = DecodeEngine(model, max_len=ctx + 8 + 2 * n_it * 4)
+
+                        def one():
+                            eng.set_state(5, ctx)
+                            eng.step()
+                        t = clock(one, n_it)
+                    else:
+                        eng = ContinuousBatcher(model, max_batch=B, max_len=ctx + 8)
+                        items = [Item(Request(b, [1], 1, slot=b), [b + 1], ctx) for b in range(B)]
+                        t = clock(lambda: eng._graph_step(items, sync=False), n_it)
+                    r["decode"].append({"batch": B, "context": ctx, "ms_per_step": round(t * 1e3, 4), "tokens_per_s": round(B / t, 1)})
+                    del eng
+                    torch.cuda.empty_cache()
+            del model
+            torch.cuda.empty_cache()
+        out.append(row)
+    return out
+
+
 def parse(argv=None):
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -85,6 +180,11 @@ def parse(argv=None):
     ap.add_argument("--deadline", type=float, default=1500.0,
                     help="seconds after the headline measurement at which rank 0 prints the JSON line with whatever legs have finished "
                          "(field `incomplete`) and every rank exits: a hung secondary leg (a collective that never returns) cannot suppress the line")
+    ap.add_argument("--hybrid", nargs="?", const="all", choices=["all", "prefill", "decode"],
+                    help="measure the hybrid decoders (Lebepel) beside the 1-bit LLaMA of equal size INSTEAD of the default workload: prefill and "
+                         "decode throughput at a few sizes, one JSON line of its own")
+    ap.add_argument("--hybrid-size", default="2048,4096", help="widths for --hybrid, comma-separated (of %s)" % ", ".join(map(str, HYBRID_SIZES)))
+    ap.add_argument("--hybrid-only", action="store_true", help="--hybrid without the 1-bit LLaMA beside it (profiles)")
     ap.add_argument("--pg-timeout", type=float, default=300.0, help="process-group timeout in seconds (N > 1)")
     return ap.parse_args(argv)
 
@@ -1004,6 +1104,12 @@ class Hooks:
 def main(argv=None, hooks=None):
     args = parse(argv)
     hk = hooks or Hooks()
+    if args.hybrid:
+        dev = torch.device("cuda:0")
+        rows = measure_hybrid(dev, args.hybrid, [int(w) for w in args.hybrid_size.split(",")], beside=not args.hybrid_only)
+        print(json.dumps({"metric": "hybrid_decoder_throughput", "unit": "tokens/s", "dtype": "bf16 (lebepel) / fp16 + 1-bit weights (onebit_llama)",
+                          "data": "synthetic", "sizes": rows}))
+        return
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
         # started as a plain process: launch the N ranks ourselves (their rank 0 prints the JSON line)
         env = dict(os.environ, HSA_ENABLE_IPC_MODE_LEGACY=os.environ.get("HSA_ENABLE_IPC_MODE_LEGACY", "0"))

@@ -476,10 +476,12 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
         if constexpr (!SM) {
             if (s >= S) continue;
             const int row = (int)qrow0 + s;
+            int c0 = head * AA.vdim + 4 * g;             // (opaque: the columns' offsets are formed here, not kept through the key loop)
+            asm volatile("" : "+v"(c0));
             H16 *o = (H16 *)AA.out + ((size_t)(row >> 4) * AA.out_nkt) * 512 + (row & 15) * 8;          // fragment-major row `row`
 #pragma unroll
             for (int dt = 0; dt < DT; ++dt) {
-                const int d = 16 * dt + 4 * g, c = head * AA.vdim + d;
+                const int d = 16 * dt + 4 * g, c = c0 + 16 * dt;
                 if ((AA.vdim & 3) == 0) {
                     if (d < AA.vdim) {
                         ob_fl_bf4 ov;

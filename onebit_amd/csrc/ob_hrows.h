@@ -17,12 +17,13 @@ struct ObHNormArgs {
     int W;
 };
 
+// (the workgroup is as wide as the row allows, up to 1024 threads: at one to 64 rows its few dependent passes ARE the launch's time)
 template <typename E, int VEC>
-__global__ __launch_bounds__(256) void ob_hnorm_kernel(const ObHNormArgs A)
+__global__ __launch_bounds__(1024) void ob_hnorm_kernel(const ObHNormArgs A)
 {
-    extern __shared__ __attribute__((aligned(16))) float sm[];        // [W] row | [8] reduction
+    extern __shared__ __attribute__((aligned(16))) float sm[];        // [W] row | [16] reduction
     float *red = sm + ((A.W + 3) & ~3);
-    const int t = blockIdx.x, tid = threadIdx.x;
+    const int t = blockIdx.x, tid = threadIdx.x, stride = blockDim.x * VEC;
     const int src = A.rows ? A.rows[t] : t;
     float *xr = A.x + (size_t)src * A.W;
     const E *er = nullptr, *pr = nullptr;
@@ -31,7 +32,7 @@ __global__ __launch_bounds__(256) void ob_hnorm_kernel(const ObHNormArgs A)
         if (A.pos_embed) pr = (const E *)A.pos_embed + (size_t)max(A.row_pos[src], 0) * A.W;
     }
     float ss = 0.f;
-    for (int c = tid * VEC; c < A.W; c += 256 * VEC) {
+    for (int c = tid * VEC; c < A.W; c += stride) {
         float r[VEC];
         if (er) {
 #pragma unroll
@@ -41,10 +42,18 @@ __global__ __launch_bounds__(256) void ob_hnorm_kernel(const ObHNormArgs A)
 #pragma unroll
             for (int e = 0; e < VEC; ++e) { s[e] = 0.f; xv[e] = xr[c + e]; }
             const float *zr = A.z + (size_t)src * A.ldz + c;
-            for (int k = 0; k < A.n_split; ++k) {
+            for (int k = 0; k < A.n_split; k += 4) {                  // four splits in flight, added in order
+                float zv[4][VEC];
 #pragma unroll
-                for (int e = 0; e < VEC; ++e) s[e] += zr[e];
-                zr += A.z_split;
+                for (int j = 0; j < 4; ++j)
+#pragma unroll
+                    for (int e = 0; e < VEC; ++e) zv[j][e] = zr[(size_t)min(k + j, A.n_split - 1) * A.z_split + e];
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+                    if (k + j < A.n_split) {
+#pragma unroll
+                        for (int e = 0; e < VEC; ++e) s[e] += zv[j][e];
+                    }
             }
 #pragma unroll
             for (int e = 0; e < VEC; ++e) r[e] = xv[e] + A.mult * (A.bias ? s[e] + A.bias[c + e] : s[e]);
@@ -68,7 +77,7 @@ __global__ __launch_bounds__(256) void ob_hnorm_kernel(const ObHNormArgs A)
     ss = ob_block_sum(ss, red);
     const float rs = 1.0f / sqrtf(ss / (float)A.W + A.eps);
     E *out = (E *)A.out;
-    for (int c = tid * VEC; c < A.W; c += 256 * VEC) {
+    for (int c = tid * VEC; c < A.W; c += stride) {
         ob_float4 v;
 #pragma unroll
         for (int e = 0; e < VEC; ++e) v[e] = sm[c + e] * rs * (A.off + A.w[c + e]);
@@ -123,9 +132,22 @@ __global__ __launch_bounds__(1024) void ob_argmax_rows_kernel(const float *__res
     const int tid = threadIdx.x;
     float best = -INFINITY;
     int idx = 0x7fffffff;
-    for (int i = tid; i < V; i += 1024) {
-        const float v = l[i];
-        if (v > best) { best = v; idx = i; }
+    if ((V & 3) == 0) {
+        for (int i0 = tid; i0 < V / 4; i0 += 4096) {                  // four 16-byte loads in flight
+            ob_float4 v[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[j] = reinterpret_cast<const ob_float4 *>(l)[min(i0 + 1024 * j, V / 4 - 1)];
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+#pragma unroll
+                for (int e = 0; e < 4; ++e)                           // (ascending indices; a clamped repeat is not larger)
+                    if (v[j][e] > best) { best = v[j][e]; idx = 4 * min(i0 + 1024 * j, V / 4 - 1) + e; }
+        }
+    } else {
+        for (int i = tid; i < V; i += 1024) {
+            const float v = l[i];
+            if (v > best) { best = v; idx = i; }
+        }
     }
 #pragma unroll
     for (int s = 32; s > 0; s >>= 1) {

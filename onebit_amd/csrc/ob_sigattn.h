@@ -43,6 +43,39 @@ __global__ __launch_bounds__(256) void ob_sig_prep_kernel(const ObSigPrepArgs A)
     for (int d = lane; d < np; d += 64) dst[d] = d < n ? (E)((float)src[d] * f) : (E)0.f;
 }
 
+// the same for bf16 heads of whole 16-byte pieces (dim % 8 == vdim % 8 == 0), padded to DP: DP / 8 lanes per head, one piece each
+template <int DP>
+__global__ __launch_bounds__(256) void ob_sig_prep_vec_kernel(const ObSigPrepArgs A)
+{
+    constexpr int LPH = DP / 8;
+    const int i = blockIdx.x * 256 + threadIdx.x, unit = i / LPH, ds = i % LPH, row = A.row0 + blockIdx.y;
+    const int slot = A.row_slot[row], pos = A.row_pos[row];
+    if (slot < 0 || slot >= A.n_slots || pos < 0 || pos >= A.max_len) return;                          // (uniform)
+    const bool live = unit < A.H + 2 * A.G;
+    const int kind = unit < A.H ? 0 : unit < A.H + A.G ? 1 : 2, h = kind == 0 ? unit : kind == 1 ? unit - A.H : unit - A.H - A.G;
+    const int n = kind == 2 ? A.vdim : A.dim;
+    ob_bf8 v = (ob_bf8)(__bf16)0.f;
+    if (live && 8 * ds < n)
+        v = *reinterpret_cast<const ob_bf8 *>((const __bf16 *)A.u + (size_t)row * A.ldu +
+                                              (kind < 2 ? unit * A.dim : (A.H + A.G) * A.dim + h * A.vdim) + 8 * ds);
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss = __builtin_fmaf((float)v[e], (float)v[e], ss);
+    ss += OB_DPP_F(ss, 0xB1, 0xF);
+    ss += OB_DPP_F(ss, 0x4E, 0xF);
+    ss += OB_DPP_F(ss, 0x141, 0xF);
+    if (LPH == 16) ss += OB_DPP_F(ss, 0x140, 0xF);
+    if (kind < 2 && A.unit_rms) {
+        const float f = 1.0f / sqrtf(ss / (float)n + A.eps);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = (__bf16)((float)v[e] * f);
+    }
+    if (!live) return;
+    __bf16 *dst = kind == 0 ? (__bf16 *)A.qn + ((size_t)row * A.H + h) * DP
+                            : (__bf16 *)(kind == 1 ? A.kc : A.vc) + (((size_t)slot * A.G + h) * A.max_len + pos) * DP;
+    *reinterpret_cast<ob_bf8 *>(dst + 8 * ds) = v;
+}
+
 // ---- any element type / head size: one workgroup per (row, head), fp32 arithmetic with the accurate functions
 struct ObSigRowsArgs {
     const void *qn, *kc, *vc;

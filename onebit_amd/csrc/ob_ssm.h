@@ -71,6 +71,56 @@ __global__ __launch_bounds__(256) void ob_conv_kernel(const ObSsmArgs A, const i
     else o[0] = r[0];
 }
 
+// the same for 2 to 4 taps: OB_CONV_ROWS rows per thread, the window of inputs sliding through registers (rebuilt where a run starts)
+#define OB_CONV_ROWS 8
+template <typename E, int TAPS>
+__global__ __launch_bounds__(256) void ob_conv_rows_kernel(const ObSsmArgs A, const int32_t *__restrict__ row_off, void *xbc, int row_end)
+{
+    typedef typename ObElem<E>::V16 V16;
+    constexpr int VEC = ObElem<E>::EPL, R = OB_CONV_ROWS;
+    const int row0 = A.row0 + blockIdx.y * R, c = (blockIdx.x * 256 + threadIdx.x) * VEC;
+    if (c >= A.ch) return;
+    const E *u = (const E *)A.u + A.x_off + c;
+    V16 in[R + TAPS - 1];                                          // in[TAPS - 1 + r] = row row0 + r
+#pragma unroll
+    for (int r = 0; r < R; ++r) in[TAPS - 1 + r] = *reinterpret_cast<const V16 *>(u + (size_t)min(row0 + r, row_end - 1) * A.ldu);
+    float w[TAPS][VEC], b[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) b[e] = A.conv_b[c + e];
+#pragma unroll
+    for (int t = 0; t < TAPS; ++t)
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) w[t][e] = A.conv_w[(size_t)t * A.ch + c + e];
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+        const int row = row0 + r;
+        if (row >= row_end) break;
+        const int off = row_off[row];
+        V16 x[TAPS];                                               // x[t]: TAPS - 1 - t tokens back
+#pragma unroll
+        for (int t = 0; t < TAPS; ++t) x[t] = in[r + t];
+        if (off < TAPS - 1 || r < TAPS - 1) {                      // (uniform) some of the window lies before the run or the thread's rows
+            const int slot = A.row_slot[row], pos = A.row_pos[row];
+#pragma unroll
+            for (int t = 0; t < TAPS - 1; ++t) {
+                const int back = TAPS - 1 - t;
+                if (back > pos) x[t] = (V16)(E)0.f;
+                else if (back > off) x[t] = *reinterpret_cast<const V16 *>((const E *)A.ring + ((size_t)slot * A.taps + (pos - back) % A.taps) * A.ch + c);
+                else if (r < back) x[t] = *reinterpret_cast<const V16 *>(u + (size_t)(row - back) * A.ldu);
+            }
+        }
+        V16 o;
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) {
+            float acc = b[e];
+#pragma unroll
+            for (int t = TAPS - 1; t >= 0; --t) acc = __builtin_fmaf(w[t][e], (float)x[t][e], acc);
+            o[e] = (E)ob_silu<E>(acc);
+        }
+        *reinterpret_cast<V16 *>((E *)xbc + (size_t)row * A.ldxbc + c) = o;
+    }
+}
+
 // ---- token by token.  Thread = (4 state columns, every 32nd state row): NI rows in registers
 template <typename E, int NI>
 __global__ __launch_bounds__(256) void ob_ssm_step_kernel(const ObSsmArgs A, const ObSsmSegs SG)
@@ -168,7 +218,7 @@ __global__ __launch_bounds__(256) void ob_ssd_kernel(const ObSsmArgs A, const Ob
     typedef __attribute__((address_space(3))) ob_v4s ob_lds_v4s;
     constexpr int Q = 64, LD = NP + 8, LX = 40, KN = NP / 32, NT = NP / 32;     // n tiles per wave: NP / 16 / 2
     __shared__ __attribute__((aligned(16))) __bf16 Bs[Q][LD], Cs[Q][LD], Xs[Q][LX], Sh[32][LD], Sl[32][LD];
-    __shared__ __attribute__((aligned(16))) float cum[Q], dts[Q], wgt[Q];
+    __shared__ __attribute__((aligned(16))) float cum2[2][Q], dts2[2][Q], wgt2[2][Q];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, g4 = lane >> 4;
     const int nsl = (A.P + 31) >> 5, h = blockIdx.x / nsl, p0 = (blockIdx.x % nsl) * 32, npx = min(32, A.P - p0);
     const ObSsmSeg sg = SG.s[blockIdx.y];
@@ -223,9 +273,21 @@ __global__ __launch_bounds__(256) void ob_ssd_kernel(const ObSsmArgs A, const Ob
         rx = piece(t0 + (tid >> 2), cx, (tid & 3) * 8, npx);
         if (tid < Q) rdt = t0 + tid < sg.n ? A.aux[(size_t)(sg.row0 + t0 + tid) * A.ldaux + h] : 0.f;
     };
+    // a chunk's step sizes, summed log decays and input weights: wave 0 (whose tokens have the fewest predecessors) forms the NEXT chunk's
+    // while the others still multiply
+    auto decays = [&](int t0, int buf) {
+        const float dt = t0 + lane < sg.n ? ob_softplusf(rdt + dtb) : 0.f;          // (no token: no decay, no input)
+        float c = na * dt;
+#pragma unroll
+        for (int s = 1; s < 64; s <<= 1) { const float o = __shfl_up(c, s); if (lane >= s) c += o; }
+        const float tot = __shfl(c, 63);
+        cum2[buf][lane] = c; dts2[buf][lane] = dt; wgt2[buf][lane] = dt * expf(tot - c);
+    };
     fetch(0);
+    if (wave == 0) decays(0, 0);
     for (int t0 = 0; t0 < sg.n; t0 += Q) {
-        // ---- this chunk's rows, decays and the state's two terms into LDS
+        const float *cum = cum2[(t0 / Q) & 1], *dts = dts2[(t0 / Q) & 1], *wgt = wgt2[(t0 / Q) & 1];
+        // ---- this chunk's rows and the state's two terms into LDS
 #pragma unroll
         for (int i = 0; i < PB; ++i) {
             const int j = tid + 256 * i;
@@ -234,14 +296,6 @@ __global__ __launch_bounds__(256) void ob_ssd_kernel(const ObSsmArgs A, const Ob
         }
         *reinterpret_cast<ob_bf8 *>(&Xs[tid >> 2][(tid & 3) * 8]) = rx;
         store_hl();
-        if (wave == 0) {
-            const float dt = t0 + lane < sg.n ? ob_softplusf(rdt + dtb) : 0.f;      // (no token: no decay, no input)
-            float c = na * dt;
-#pragma unroll
-            for (int s = 1; s < 64; s <<= 1) { const float o = __shfl_up(c, s); if (lane >= s) c += o; }
-            const float tot = __shfl(c, 63);
-            cum[lane] = c; dts[lane] = dt; wgt[lane] = dt * expf(tot - c);
-        }
         __syncthreads();
         if (t0 + Q < sg.n) fetch(t0 + Q);
         // ---- scores of this wave's 16 tokens against the tokens up to them
@@ -324,6 +378,7 @@ __global__ __launch_bounds__(256) void ob_ssd_kernel(const ObSsmArgs A, const Ob
                 S[i] = ObElem<__bf16>::mma(bt, xl, S[i]);
             }
         }
+        if (wave == 0 && t0 + Q < sg.n) decays(t0 + Q, ((t0 / Q) & 1) ^ 1);
         __syncthreads();                                         // every read of this chunk's LDS is complete
     }
 #pragma unroll

@@ -212,8 +212,9 @@ static int norm_launch(const ObHNormArgs &a, int rows, hipStream_t s)
     auto k4 = ob_hnorm_kernel<E, 4>;
     auto k1 = ob_hnorm_kernel<E, 1>;
     if (!lds_ok(a.W % 4 == 0 ? (const void *)k4 : (const void *)k1, lds)) return hfail(ONEBIT_E_SHAPE, "norm: LDS");
-    if (a.W % 4 == 0) hipLaunchKernelGGL(k4, dim3((unsigned)rows), dim3(256), lds, s, a);
-    else hipLaunchKernelGGL(k1, dim3((unsigned)rows), dim3(256), lds, s, a);
+    const unsigned thr = (unsigned)std::min<int64_t>(rows <= 256 ? 1024 : 512, std::max<int64_t>(64, rup(cdiv(a.W, 4), 64)));
+    if (a.W % 4 == 0) hipLaunchKernelGGL(k4, dim3((unsigned)rows), dim3(thr), lds, s, a);
+    else hipLaunchKernelGGL(k1, dim3((unsigned)rows), dim3(thr), lds, s, a);
     return hstatus("norm");
 }
 
@@ -241,6 +242,14 @@ static int attention_launch(const onebit_hmodel_t &m, const onebit_hlayer_t &L, 
     for (int r0 = 0; r0 < rest; r0 += 32768) {                       // (grid y limit)
         ObSigPrepArgs pp = p;
         pp.row0 = n_dec + r0;
+        if constexpr (sizeof(E) == 2) {
+            if (mfma && L.dim % 8 == 0 && L.vdim % 8 == 0) {
+                const dim3 grid((unsigned)cdiv((int64_t)(L.heads + 2 * L.kv_heads) * (L.kp / 8), 256), (unsigned)std::min(rest - r0, 32768));
+                if (L.kp == 64) hipLaunchKernelGGL((ob_sig_prep_vec_kernel<64>), grid, dim3(256), 0, s, pp);
+                else hipLaunchKernelGGL((ob_sig_prep_vec_kernel<128>), grid, dim3(256), 0, s, pp);
+                continue;
+            }
+        }
         hipLaunchKernelGGL((ob_sig_prep_kernel<E>), dim3((unsigned)cdiv(L.heads + 2 * L.kv_heads, 4), (unsigned)std::min(rest - r0, 32768)), dim3(256), 0, s, pp);
     }
     if (int rc = hstatus("attention inputs")) return rc;
@@ -301,7 +310,13 @@ static int ssm_launch(const onebit_hmodel_t &m, const onebit_hlayer_t &L, const 
             ObSsmArgs c = a;
             c.row0 = st.n_dec + r0;
             const unsigned ny = (unsigned)std::min(rest - r0, 32768);
-            if (ch % VEC == 0 && inner % VEC == 0) hipLaunchKernelGGL((ob_conv_kernel<E, VEC>), dim3((unsigned)cdiv(ch / VEC, 256), ny), dim3(256), 0, s, c, st.row_off, ws + P.xbc);
+            if (ch % VEC == 0 && inner % VEC == 0 && L.taps >= 2 && L.taps <= 4) {
+                const dim3 grid((unsigned)cdiv(ch / VEC, 256), (unsigned)cdiv(ny, OB_CONV_ROWS));
+                const int last = st.n_dec + r0 + (int)ny;
+                if (L.taps == 2) hipLaunchKernelGGL((ob_conv_rows_kernel<E, 2>), grid, dim3(256), 0, s, c, st.row_off, ws + P.xbc, last);
+                else if (L.taps == 3) hipLaunchKernelGGL((ob_conv_rows_kernel<E, 3>), grid, dim3(256), 0, s, c, st.row_off, ws + P.xbc, last);
+                else hipLaunchKernelGGL((ob_conv_rows_kernel<E, 4>), grid, dim3(256), 0, s, c, st.row_off, ws + P.xbc, last);
+            } else if (ch % VEC == 0 && inner % VEC == 0) hipLaunchKernelGGL((ob_conv_kernel<E, VEC>), dim3((unsigned)cdiv(ch / VEC, 256), ny), dim3(256), 0, s, c, st.row_off, ws + P.xbc);
             else hipLaunchKernelGGL((ob_conv_kernel<E, 1>), dim3((unsigned)cdiv(ch, 256), ny), dim3(256), 0, s, c, st.row_off, ws + P.xbc);
         }
         if (int rc = hstatus("convolution")) return rc;

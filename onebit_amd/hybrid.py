@@ -399,7 +399,7 @@ class HybridStep:
     def _launch_graph(self, items):
         B, V = self.n_slots, self.model.vocab_size
         n = len(items)
-        if n > B or len({it[0] for it in items}) != n:
+        if not 0 < n <= B or len({it[0] for it in items}) != n:
             raise ValueError(f"step: {n} items for {B} slots, or a repeated slot")
         ctx = 0
         for i, (slot, start, toks) in enumerate(it[:3] for it in items):
