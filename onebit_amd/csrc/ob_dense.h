@@ -46,6 +46,16 @@ template <typename E> __device__ __forceinline__ ob_float4 ob_load4f(const E *p)
     return (ob_float4){(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
 }
 
+// two floats as bf16 pairs hi + lo: hi = the upper halves (truncated), lo = what is left, rounded -- 16 bits of mantissa together
+typedef __bf16 ob_bf2 __attribute__((ext_vector_type(2)));
+__device__ __forceinline__ uint32_t ob_pack_bf2(float a, float b) { return __builtin_bit_cast(uint32_t, __builtin_convertvector((ob_float2){a, b}, ob_bf2)); }
+__device__ __forceinline__ void ob_split_bf2(float a, float b, uint32_t &hi, uint32_t &lo)
+{
+    const uint32_t ua = __float_as_uint(a), ub = __float_as_uint(b);
+    hi = __builtin_amdgcn_perm(ub, ua, 0x07060302u);
+    lo = ob_pack_bf2(a - __uint_as_float(ua & 0xffff0000u), b - __uint_as_float(ub & 0xffff0000u));
+}
+
 // element offset of (row, k) in a fragment-major matrix with nkt tiles per 16-row band
 template <typename E> __host__ __device__ __forceinline__ size_t ob_frag(int row, int k, int nkt)
 {

@@ -92,21 +92,22 @@ struct ObGatedNormArgs {
     const float *w; float eps; int gsize;
     void *out; int out_nkt;
 };
-template <typename E, int VEC>
+template <typename E, int VEC>                                 // VEC = 16 bytes of elements, or 1
 __global__ __launch_bounds__(256) void ob_gated_norm_kernel(const ObGatedNormArgs A)
 {
+    typedef typename ObElem<E>::V16 V16;
     extern __shared__ __attribute__((aligned(16))) float sm[];
     float *red = sm + ((A.gsize + 3) & ~3);
-    const int t = blockIdx.y, c0 = blockIdx.x * A.gsize, tid = threadIdx.x;
+    const int t = blockIdx.y, c0 = blockIdx.x * A.gsize, tid = threadIdx.x, stride = blockDim.x * VEC;
     const E *y = (const E *)A.y + (size_t)t * A.ldy + c0, *z = (const E *)A.gate + (size_t)t * A.ldg + c0;
     float ss = 0.f;
-    for (int c = tid * VEC; c < A.gsize; c += 256 * VEC) {
-        ob_float4 yv, zv;
-        if constexpr (VEC == 4) { yv = ob_load4f(y + c); zv = ob_load4f(z + c); }
-        else { yv[0] = (float)y[c]; zv[0] = (float)z[c]; }
+    for (int c = tid * VEC; c < A.gsize; c += stride) {
+        V16 yv, zv;
+        if constexpr (VEC > 1) { yv = *reinterpret_cast<const V16 *>(y + c); zv = *reinterpret_cast<const V16 *>(z + c); }
+        else { yv[0] = y[c]; zv[0] = z[c]; }
 #pragma unroll
         for (int e = 0; e < VEC; ++e) {
-            const float v = yv[e] * ob_silu<E>(zv[e]);
+            const float v = (float)yv[e] * ob_silu<E>((float)zv[e]);
             sm[c + e] = v;
             ss = __builtin_fmaf(v, v, ss);
         }
@@ -114,12 +115,12 @@ __global__ __launch_bounds__(256) void ob_gated_norm_kernel(const ObGatedNormArg
     ss = ob_block_sum(ss, red);
     const float rs = 1.0f / sqrtf(ss / (float)A.gsize + A.eps);
     E *out = (E *)A.out;
-    for (int c = tid * VEC; c < A.gsize; c += 256 * VEC) {
-        ob_float4 v;
+    for (int c = tid * VEC; c < A.gsize; c += stride) {
+        V16 v;
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) v[e] = sm[c + e] * rs * A.w[c0 + c + e];
-        if constexpr (VEC == 4) *reinterpret_cast<typename ObElem<E>::V4 *>(out + ob_frag<E>(t, c0 + c, A.out_nkt)) = ob_to_v4<E>(v);
-        else out[ob_frag<E>(t, c0 + c, A.out_nkt)] = (E)v[0];
+        for (int e = 0; e < VEC; ++e) v[e] = (E)(sm[c + e] * rs * A.w[c0 + c + e]);
+        if constexpr (VEC > 1) *reinterpret_cast<V16 *>(out + ob_frag<E>(t, c0 + c, A.out_nkt)) = v;       // (16 bytes of a row are contiguous)
+        else out[ob_frag<E>(t, c0 + c, A.out_nkt)] = v[0];
     }
 }
 

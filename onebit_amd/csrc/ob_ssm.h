@@ -210,14 +210,27 @@ __global__ __launch_bounds__(256) void ob_ssm_step_kernel(const ObSsmArgs A, con
 // ---- chunks of 64 tokens on MFMA (bf16 x / B / C).  Workgroup = (segment, head, 32 state columns), 4 waves; NP = N padded.
 //   G^T[s][t] = B_s . C_t (wave w: tokens 16 w ..), masked and decayed in registers -> it IS the B operand of Y^T += X^T M^T
 //   Y^T[p][t] = (S_prev^T C_t) exp(cum_t) + X^T M^T + D x;   S <- exp(cum_63) S + B^T (x dt exp(cum_63 - cum))
+// The kernel is bound by VALU issue (two waves per SIMD): decays live in the base-2 domain, the weighted inputs x dt exp(..) are formed once
+// per element on their way into LDS, splits into bf16 terms cost three operations per element, tiles above the diagonal none.
+// LDS rows of 128 / 256 columns are unpadded, 16-byte pieces XOR-swizzled by the row: piece pc of row r sits at pc ^ f(r), f(r) = 2 m + (r >> 3),
+// m = r for rows 0 .. 7 and (r - 8) ^ 4 for rows 8 .. 15.  Operand reads (a ds_read_b128 lane group = rows {0-3, 12-15} at one piece and rows
+// 4-11 at the next) and transpose reads (a half-wave = two adjacent pieces of 8 rows) then both cover the 64 banks once.
+template <int NP> __device__ __forceinline__ int ob_ssd_at(int r, int k)      // element offset of (row, column) in such a tile
+{
+    if constexpr (NP < 128) return r * (NP + 8) + k;                          // (64 columns: padded rows)
+    else {
+        const int r16 = r & 15, f = 2 * (r16 < 8 ? r16 : (r16 & 7) ^ 4) + (r16 >> 3);
+        return r * NP + ((((k >> 3) ^ f) << 3) | (k & 7));
+    }
+}
 template <int NP, bool VEC>
 __global__ __launch_bounds__(256) void ob_ssd_kernel(const ObSsmArgs A, const ObSsmSegs SG)
 {
     typedef short ob_v4s __attribute__((ext_vector_type(4)));
     typedef short ob_v8s __attribute__((ext_vector_type(8)));
     typedef __attribute__((address_space(3))) ob_v4s ob_lds_v4s;
-    constexpr int Q = 64, LD = NP + 8, LX = 40, KN = NP / 32, NT = NP / 32;     // n tiles per wave: NP / 16 / 2
-    __shared__ __attribute__((aligned(16))) __bf16 Bs[Q][LD], Cs[Q][LD], Xs[Q][LX], Sh[32][LD], Sl[32][LD];
+    constexpr int Q = 64, LD = NP < 128 ? NP + 8 : NP, LX = 48, KN = NP / 32, NT = NP / 32;     // n tiles per wave: NP / 16 / 2
+    __shared__ __attribute__((aligned(16))) __bf16 Bs[Q * LD], Cs[Q * LD], Xs[Q][LX], Xh[Q][LX], Xl[Q][LX], Sh[32 * LD], Sl[32 * LD];
     __shared__ __attribute__((aligned(16))) float cum2[2][Q], dts2[2][Q], wgt2[2][Q];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, g4 = lane >> 4;
     const int nsl = (A.P + 31) >> 5, h = blockIdx.x / nsl, p0 = (blockIdx.x % nsl) * 32, npx = min(32, A.P - p0);
@@ -225,21 +238,11 @@ __global__ __launch_bounds__(256) void ob_ssd_kernel(const ObSsmArgs A, const Ob
     const int grp = h / (A.heads / A.groups), inner = A.heads * A.P, GN = A.groups * A.N;
     const __bf16 *xb = (const __bf16 *)A.xbc + (size_t)sg.row0 * A.ldxbc;
     const int cx = h * A.P + p0, cB = inner + grp * A.N, cC = inner + GN + grp * A.N;
-    const float dtb = A.dt_bias[h], na = -expf(A.A_log[h]), Dh = A.D[h];
+    const float dtb = A.dt_bias[h], na = -1.4426950408889634f * expf(A.A_log[h]), Dh = A.D[h];
     float *st = A.state + (((size_t)sg.slot * A.heads + h) * A.N) * A.sp;
     // state: wave = (p tile wave & 1, n tiles (wave >> 1) NT ..); lane holds column p = lr, rows n = 4 g4 .. + 3
     const int pt = wave & 1, nt0 = (wave >> 1) * NT, pcol = p0 + 16 * pt + lr;
     ob_float4 S[NT];
-    auto store_hl = [&]() {
-#pragma unroll
-        for (int i = 0; i < NT; ++i) {
-            ob_bf4 hi, lo;
-#pragma unroll
-            for (int e = 0; e < 4; ++e) { hi[e] = (__bf16)S[i][e]; lo[e] = (__bf16)(S[i][e] - (float)hi[e]); }
-            *reinterpret_cast<ob_bf4 *>(&Sh[16 * pt + lr][16 * (nt0 + i) + 4 * g4]) = hi;
-            *reinterpret_cast<ob_bf4 *>(&Sl[16 * pt + lr][16 * (nt0 + i) + 4 * g4]) = lo;
-        }
-    };
 #pragma unroll
     for (int i = 0; i < NT; ++i)
 #pragma unroll
@@ -247,33 +250,38 @@ __global__ __launch_bounds__(256) void ob_ssd_kernel(const ObSsmArgs A, const Ob
             const int n = 16 * (nt0 + i) + 4 * g4 + e;
             S[i][e] = sg.past > 0 && n < A.N && pcol < A.P ? st[(size_t)n * A.sp + pcol] : 0.f;
         }
-    // staging: pieces of 8 channels; rows past the run and channels past N / P are zero
-    constexpr int NPC = NP / 8, PB = Q * NPC / 256;             // pieces of B (and C) per thread; X: one piece per thread (64 x 4)
-    ob_bf8 rb[PB], rc[PB], rx;
+    // staging: pieces of 8 channels; rows past the run and channels past N / P are zero.  Thread: piece kp of rows tb + RB i of B and of C
+    constexpr int NPC = NP / 8, PB = Q * NPC / 256, RB = 256 / NPC;
+    const int tb = tid / NPC, kb = (tid % NPC) * 8, tx = tid >> 2, kx = (tid & 3) * 8;
+    ob_u32x4 rb[PB], rc[PB], rx;
     float rdt = 0.f;
-    auto piece = [&](int t, int col, int k, int n) {            // 8 channels col + k .. of token t, of which n exist
-        ob_bf8 v = (ob_bf8)(__bf16)0.f;
-        if (t < sg.n && k < n) {
-            const __bf16 *s = xb + (size_t)t * A.ldxbc + col + k;
-            if constexpr (VEC) v = *reinterpret_cast<const ob_bf8 *>(s);
+    auto piece = [&](const __bf16 *s, bool in, int k, int n) {           // 8 channels from s, of which n - k exist
+        ob_u32x4 v = {0u, 0u, 0u, 0u};
+        if (in && k < n) {
+            if constexpr (VEC) v = *reinterpret_cast<const ob_u32x4 *>(s);
             else {
+                ob_bf8 w = (ob_bf8)(__bf16)0.f;
 #pragma unroll
-                for (int e = 0; e < 8; ++e) if (k + e < n) v[e] = s[e];
+                for (int e = 0; e < 8; ++e) if (k + e < n) w[e] = s[e];
+                v = __builtin_bit_cast(ob_u32x4, w);
             }
         }
         return v;
     };
-    auto fetch = [&](int t0) {
+    const __bf16 *sB = xb + (size_t)tb * A.ldxbc + cB + kb, *sC = sB + (cC - cB), *sX = xb + (size_t)tx * A.ldxbc + cx + kx;
+    const float *sD = A.aux + (size_t)(sg.row0 + lane) * A.ldaux + h;
+    auto fetch = [&](int t0) {                                            // (called once per chunk, in order: the pointers advance)
 #pragma unroll
         for (int i = 0; i < PB; ++i) {
-            const int j = tid + 256 * i, t = t0 + j / NPC, k = (j % NPC) * 8;
-            rb[i] = piece(t, cB, k, A.N);
-            rc[i] = piece(t, cC, k, A.N);
+            const bool in = t0 + tb + RB * i < sg.n;
+            rb[i] = piece(sB + (size_t)(RB * i) * A.ldxbc, in, kb, A.N);
+            rc[i] = piece(sC + (size_t)(RB * i) * A.ldxbc, in, kb, A.N);
         }
-        rx = piece(t0 + (tid >> 2), cx, (tid & 3) * 8, npx);
-        if (tid < Q) rdt = t0 + tid < sg.n ? A.aux[(size_t)(sg.row0 + t0 + tid) * A.ldaux + h] : 0.f;
+        rx = piece(sX, t0 + tx < sg.n, kx, npx);
+        if (wave == 0) rdt = t0 + lane < sg.n ? *sD : 0.f;
+        sB += (size_t)Q * A.ldxbc; sC += (size_t)Q * A.ldxbc; sX += (size_t)Q * A.ldxbc; sD += (size_t)Q * A.ldaux;
     };
-    // a chunk's step sizes, summed log decays and input weights: wave 0 (whose tokens have the fewest predecessors) forms the NEXT chunk's
+    // a chunk's step sizes, summed log2 decays and input weights: wave 0 (whose tokens have the fewest predecessors) forms the NEXT chunk's
     // while the others still multiply
     auto decays = [&](int t0, int buf) {
         const float dt = t0 + lane < sg.n ? ob_softplusf(rdt + dtb) : 0.f;          // (no token: no decay, no input)
@@ -281,99 +289,127 @@ __global__ __launch_bounds__(256) void ob_ssd_kernel(const ObSsmArgs A, const Ob
 #pragma unroll
         for (int s = 1; s < 64; s <<= 1) { const float o = __shfl_up(c, s); if (lane >= s) c += o; }
         const float tot = __shfl(c, 63);
-        cum2[buf][lane] = c; dts2[buf][lane] = dt; wgt2[buf][lane] = dt * expf(tot - c);
+        cum2[buf][lane] = c; dts2[buf][lane] = dt; wgt2[buf][lane] = dt * __builtin_amdgcn_exp2f(tot - c);
     };
     fetch(0);
     if (wave == 0) decays(0, 0);
+    __syncthreads();
+    auto tr8 = [&](const __bf16 *lo_p, const __bf16 *hi_p) {             // two transpose reads: 4 + 4 rows of this lane's column
+        const ob_v4s lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((ob_lds_v4s *)lo_p);
+        const ob_v4s hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((ob_lds_v4s *)hi_p);
+        return __builtin_bit_cast(ob_bf8, (ob_v8s){lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
+    };
+    const int trow = 4 * g4 + (lr >> 2), tcol = 4 * (lr & 3);
     for (int t0 = 0; t0 < sg.n; t0 += Q) {
         const float *cum = cum2[(t0 / Q) & 1], *dts = dts2[(t0 / Q) & 1], *wgt = wgt2[(t0 / Q) & 1];
-        // ---- this chunk's rows and the state's two terms into LDS
+        // ---- this chunk's rows, its weighted inputs and the state's two terms into LDS
 #pragma unroll
         for (int i = 0; i < PB; ++i) {
-            const int j = tid + 256 * i;
-            *reinterpret_cast<ob_bf8 *>(&Bs[j / NPC][(j % NPC) * 8]) = rb[i];
-            *reinterpret_cast<ob_bf8 *>(&Cs[j / NPC][(j % NPC) * 8]) = rc[i];
+            *reinterpret_cast<ob_u32x4 *>(&Bs[ob_ssd_at<NP>(tb + RB * i, kb)]) = rb[i];
+            *reinterpret_cast<ob_u32x4 *>(&Cs[ob_ssd_at<NP>(tb + RB * i, kb)]) = rc[i];
         }
-        *reinterpret_cast<ob_bf8 *>(&Xs[tid >> 2][(tid & 3) * 8]) = rx;
-        store_hl();
+        *reinterpret_cast<ob_u32x4 *>(&Xs[tx][kx]) = rx;
+        {
+            const float w = wgt[tx];
+            ob_u32x4 xh, xl;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                uint32_t hi, lo;
+                ob_split_bf2(__uint_as_float(rx[e] << 16) * w, __uint_as_float(rx[e] & 0xffff0000u) * w, hi, lo);
+                xh[e] = hi; xl[e] = lo;
+            }
+            *reinterpret_cast<ob_u32x4 *>(&Xh[tx][kx]) = xh;
+            *reinterpret_cast<ob_u32x4 *>(&Xl[tx][kx]) = xl;
+        }
+#pragma unroll
+        for (int i = 0; i < NT; ++i) {
+            uint32_t h0, l0, h1, l1;
+            ob_split_bf2(S[i][0], S[i][1], h0, l0);
+            ob_split_bf2(S[i][2], S[i][3], h1, l1);
+            *reinterpret_cast<ob_u32x2 *>(&Sh[ob_ssd_at<NP>(16 * pt + lr, 16 * (nt0 + i) + 4 * g4)]) = (ob_u32x2){h0, h1};
+            *reinterpret_cast<ob_u32x2 *>(&Sl[ob_ssd_at<NP>(16 * pt + lr, 16 * (nt0 + i) + 4 * g4)]) = (ob_u32x2){l0, l1};
+        }
         __syncthreads();
         if (t0 + Q < sg.n) fetch(t0 + Q);
         // ---- scores of this wave's 16 tokens against the tokens up to them
         ob_bf8 cf[KN];
 #pragma unroll
-        for (int k = 0; k < KN; ++k) cf[k] = *reinterpret_cast<const ob_bf8 *>(&Cs[16 * wave + lr][32 * k + 8 * g4]);
+        for (int k = 0; k < KN; ++k) cf[k] = *reinterpret_cast<const ob_bf8 *>(&Cs[ob_ssd_at<NP>(16 * wave + lr, 32 * k + 8 * g4)]);
         const int tq = 16 * wave + lr;
         const float ct = cum[tq];
-        ob_bf8 mh[2], ml[2];
+        ob_u32x4 mh[2], ml[2];
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            ob_float4 a = {0.f, 0.f, 0.f, 0.f};
+            uint32_t h0 = 0, l0 = 0, h1 = 0, l1 = 0;
             if (j <= wave) {                                     // (wave-uniform)
+                ob_float4 a = {0.f, 0.f, 0.f, 0.f}, a1 = {0.f, 0.f, 0.f, 0.f};          // (two chains: a dependent MFMA waits for its predecessor)
 #pragma unroll
-                for (int k = 0; k < KN; ++k)
-                    a = ObElem<__bf16>::mma(*reinterpret_cast<const ob_bf8 *>(&Bs[16 * j + lr][32 * k + 8 * g4]), cf[k], a);
-            }
-            const ob_float4 cs = *reinterpret_cast<const ob_float4 *>(&cum[16 * j + 4 * g4]), ds = *reinterpret_cast<const ob_float4 *>(&dts[16 * j + 4 * g4]);
+                for (int k = 0; k < KN; k += 2) {
+                    a = ObElem<__bf16>::mma(*reinterpret_cast<const ob_bf8 *>(&Bs[ob_ssd_at<NP>(16 * j + lr, 32 * k + 8 * g4)]), cf[k], a);
+                    a1 = ObElem<__bf16>::mma(*reinterpret_cast<const ob_bf8 *>(&Bs[ob_ssd_at<NP>(16 * j + lr, 32 * k + 32 + 8 * g4)]), cf[k + 1], a1);
+                }
+                a += a1;
+                const ob_float4 cs = *reinterpret_cast<const ob_float4 *>(&cum[16 * j + 4 * g4]), ds = *reinterpret_cast<const ob_float4 *>(&dts[16 * j + 4 * g4]);
+                float m[4];
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const float m = 16 * j + 4 * g4 + e <= tq ? a[e] * (ds[e] * __builtin_amdgcn_exp2f((ct - cs[e]) * 1.4426950408889634f)) : 0.f;
-                const __bf16 hi = (__bf16)m;
-                mh[j >> 1][4 * (j & 1) + e] = hi;
-                ml[j >> 1][4 * (j & 1) + e] = (__bf16)(m - (float)hi);
+                for (int e = 0; e < 4; ++e) {
+                    m[e] = a[e] * (ds[e] * __builtin_amdgcn_exp2f(ct - cs[e]));
+                    if (j == wave && 4 * g4 + e > lr) m[e] = 0.f;
+                }
+                ob_split_bf2(m[0], m[1], h0, l0);
+                ob_split_bf2(m[2], m[3], h1, l1);
             }
+            mh[j >> 1][2 * (j & 1)] = h0; mh[j >> 1][2 * (j & 1) + 1] = h1;
+            ml[j >> 1][2 * (j & 1)] = l0; ml[j >> 1][2 * (j & 1) + 1] = l1;
         }
         // ---- outputs
-        const float ec = expf(ct);
+        const float ec = __builtin_amdgcn_exp2f(ct);
+        ob_float4 ya[2][2];                                      // [p tile][hi, lo]: four independent chains
+#pragma unroll
+        for (int q = 0; q < 2; ++q) ya[q][0] = ya[q][1] = (ob_float4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int k = 0; k < KN; ++k)
+#pragma unroll
+            for (int q = 0; q < 2; ++q) {
+                ya[q][0] = ObElem<__bf16>::mma(*reinterpret_cast<const ob_bf8 *>(&Sh[ob_ssd_at<NP>(16 * q + lr, 32 * k + 8 * g4)]), cf[k], ya[q][0]);
+                ya[q][1] = ObElem<__bf16>::mma(*reinterpret_cast<const ob_bf8 *>(&Sl[ob_ssd_at<NP>(16 * q + lr, 32 * k + 8 * g4)]), cf[k], ya[q][1]);
+            }
+#pragma unroll
+        for (int q = 0; q < 2; ++q) { ya[q][0] *= ec; ya[q][1] *= ec; }
+#pragma unroll
+        for (int s = 0; s < 2; ++s) {
+            if (2 * s > wave) continue;
+#pragma unroll
+            for (int q = 0; q < 2; ++q) {
+                const ob_bf8 xt = tr8(&Xs[32 * s + trow][16 * q + tcol], &Xs[32 * s + 16 + trow][16 * q + tcol]);
+                ya[q][0] = ObElem<__bf16>::mma(xt, __builtin_bit_cast(ob_bf8, mh[s]), ya[q][0]);
+                ya[q][1] = ObElem<__bf16>::mma(xt, __builtin_bit_cast(ob_bf8, ml[s]), ya[q][1]);
+            }
+        }
 #pragma unroll
         for (int q = 0; q < 2; ++q) {
-            ob_float4 y = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-            for (int k = 0; k < KN; ++k) {
-                y = ObElem<__bf16>::mma(*reinterpret_cast<const ob_bf8 *>(&Sh[16 * q + lr][32 * k + 8 * g4]), cf[k], y);
-                y = ObElem<__bf16>::mma(*reinterpret_cast<const ob_bf8 *>(&Sl[16 * q + lr][32 * k + 8 * g4]), cf[k], y);
-            }
-            y *= ec;
-#pragma unroll
-            for (int s = 0; s < 2; ++s) {
-                if (2 * s > wave) continue;
-                const ob_v4s lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((ob_lds_v4s *)(&Xs[32 * s + 4 * g4 + (lr >> 2)][16 * q + 4 * (lr & 3)]));
-                const ob_v4s hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((ob_lds_v4s *)(&Xs[32 * s + 16 + 4 * g4 + (lr >> 2)][16 * q + 4 * (lr & 3)]));
-                const ob_bf8 xt = __builtin_bit_cast(ob_bf8, (ob_v8s){lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
-                y = ObElem<__bf16>::mma(xt, mh[s], y);
-                y = ObElem<__bf16>::mma(xt, ml[s], y);
-            }
-            const ob_bf4 xv = *reinterpret_cast<const ob_bf4 *>(&Xs[tq][16 * q + 4 * g4]);
+            ob_float4 y = ya[q][0] + ya[q][1];
+            const ob_u32x2 xv = *reinterpret_cast<const ob_u32x2 *>(&Xs[tq][16 * q + 4 * g4]);
             const int p = 16 * q + 4 * g4;
             if (t0 + tq < sg.n) {
                 __bf16 *o = (__bf16 *)A.y + (size_t)(sg.row0 + t0 + tq) * A.ldy + cx + p;
 #pragma unroll
-                for (int e = 0; e < 4; ++e) y[e] = __builtin_fmaf(Dh, (float)xv[e], y[e]);
-                if constexpr (VEC) { if (p < npx) *reinterpret_cast<ob_bf4 *>(o) = ob_to_v4<__bf16>(y); }
+                for (int e = 0; e < 4; ++e) y[e] = __builtin_fmaf(Dh, __uint_as_float((e & 1) ? xv[e >> 1] & 0xffff0000u : xv[e >> 1] << 16), y[e]);
+                if constexpr (VEC) { if (p < npx) *reinterpret_cast<ob_u32x2 *>(o) = (ob_u32x2){ob_pack_bf2(y[0], y[1]), ob_pack_bf2(y[2], y[3])}; }
                 else { for (int e = 0; e < 4; ++e) if (p + e < npx) o[e] = (__bf16)y[e]; }
             }
         }
         // ---- the state behind the chunk
-        const float et = expf(cum[63]);
+        const float et = __builtin_amdgcn_exp2f(cum[63]);
 #pragma unroll
         for (int i = 0; i < NT; ++i) S[i] *= et;
 #pragma unroll
         for (int s = 0; s < 2; ++s) {
-            const ob_v4s lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((ob_lds_v4s *)(&Xs[32 * s + 4 * g4 + (lr >> 2)][16 * pt + 4 * (lr & 3)]));
-            const ob_v4s hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((ob_lds_v4s *)(&Xs[32 * s + 16 + 4 * g4 + (lr >> 2)][16 * pt + 4 * (lr & 3)]));
-            const ob_bf8 xt = __builtin_bit_cast(ob_bf8, (ob_v8s){lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
-            const ob_float4 w0 = *reinterpret_cast<const ob_float4 *>(&wgt[32 * s + 4 * g4]), w1 = *reinterpret_cast<const ob_float4 *>(&wgt[32 * s + 16 + 4 * g4]);
-            ob_bf8 xh, xl;
-#pragma unroll
-            for (int e = 0; e < 8; ++e) {
-                const float v = (float)xt[e] * (e < 4 ? w0[e & 3] : w1[e & 3]);
-                xh[e] = (__bf16)v;
-                xl[e] = (__bf16)(v - (float)xh[e]);
-            }
+            const ob_bf8 xh = tr8(&Xh[32 * s + trow][16 * pt + tcol], &Xh[32 * s + 16 + trow][16 * pt + tcol]);
+            const ob_bf8 xl = tr8(&Xl[32 * s + trow][16 * pt + tcol], &Xl[32 * s + 16 + trow][16 * pt + tcol]);
 #pragma unroll
             for (int i = 0; i < NT; ++i) {
-                const ob_v4s bl = __builtin_amdgcn_ds_read_tr16_b64_v4i16((ob_lds_v4s *)(&Bs[32 * s + 4 * g4 + (lr >> 2)][16 * (nt0 + i) + 4 * (lr & 3)]));
-                const ob_v4s bh = __builtin_amdgcn_ds_read_tr16_b64_v4i16((ob_lds_v4s *)(&Bs[32 * s + 16 + 4 * g4 + (lr >> 2)][16 * (nt0 + i) + 4 * (lr & 3)]));
-                const ob_bf8 bt = __builtin_bit_cast(ob_bf8, (ob_v8s){bl[0], bl[1], bl[2], bl[3], bh[0], bh[1], bh[2], bh[3]});
+                const ob_bf8 bt = tr8(&Bs[ob_ssd_at<NP>(32 * s + trow, 16 * (nt0 + i) + tcol)], &Bs[ob_ssd_at<NP>(32 * s + 16 + trow, 16 * (nt0 + i) + tcol)]);
                 S[i] = ObElem<__bf16>::mma(bt, xh, S[i]);
                 S[i] = ObElem<__bf16>::mma(bt, xl, S[i]);
             }

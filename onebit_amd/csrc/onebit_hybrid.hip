@@ -341,16 +341,17 @@ static int ssm_launch(const onebit_hmodel_t &m, const onebit_hlayer_t &L, const 
     }
     ObGatedNormArgs n = {ws + P.y, ldy, ws + P.u, 16 * L.nt_mix, L.gnorm_w, m.eps, inner / L.norm_groups, act, act_nkt};
     const int lds = (((n.gsize + 3) & ~3) + 16) * 4;
-    auto k4 = ob_gated_norm_kernel<E, 4>;
+    auto k4 = ob_gated_norm_kernel<E, VEC>;
     auto k1 = ob_gated_norm_kernel<E, 1>;
-    if (!lds_ok(n.gsize % 4 == 0 ? (const void *)k4 : (const void *)k1, lds)) return hfail(ONEBIT_E_SHAPE, "gated norm: LDS");
+    if (!lds_ok(n.gsize % VEC == 0 ? (const void *)k4 : (const void *)k1, lds)) return hfail(ONEBIT_E_SHAPE, "gated norm: LDS");
     for (int r0 = 0; r0 < st.n_rows; r0 += 32768) {
         // (32768 rows = a whole number of 16-row bands: the fragment-major rows of the slice start at a band)
         n.y = ws + P.y + (size_t)r0 * ldy * sizeof(E);
         n.gate = ws + P.u + (size_t)r0 * n.ldg * sizeof(E);
         n.out = (char *)act + (size_t)(r0 / 16) * act_nkt * 1024;
         const dim3 grid((unsigned)L.norm_groups, (unsigned)std::min(st.n_rows - r0, 32768));
-        if (n.gsize % 4 == 0) hipLaunchKernelGGL(k4, grid, dim3(256), lds, s, n);
+        const unsigned thr = (unsigned)std::min<int64_t>(256, std::max<int64_t>(64, rup(cdiv(n.gsize, VEC), 64)));
+        if (n.gsize % VEC == 0) hipLaunchKernelGGL(k4, grid, dim3(thr), lds, s, n);
         else hipLaunchKernelGGL(k1, grid, dim3(256), lds, s, n);
     }
     return hstatus("gated norm");
