@@ -32,6 +32,7 @@ def _load_onebit(path, device, dtype):
 
 
 def _engine_onebit(model, n_slots, max_len):
+    n_slots = max(n_slots, 32)                      # (a fixed cache: enough slots from the start)
     from .engine import MixedStep
     from .llama import KVCache
     cache = KVCache(model.config, n_slots, max_len, model.lm_head.weight.device, torch.float16)

@@ -24,7 +24,7 @@ class TraceSession:
 
     def __init__(self, family, model, max_len: int, n_slots: int = 8):
         self.engine = family.engine(model, n_slots, max_len)
-        self.pool = SlotPool(n_slots)
+        self.pool = SlotPool(self.engine.n_slots)
         self.live: Dict[str, Tuple[int, int]] = {}
 
     def step(self, entries: List[dict], end: List[str] = ()) -> Optional[torch.Tensor]:
@@ -33,6 +33,8 @@ class TraceSession:
         new = sum(e["id"] not in self.live for e in entries)
         if new > len(self.pool):
             n = max(2 * self.pool.n, self.pool.n + new - len(self.pool))
+            if not hasattr(self.engine, "grow"):
+                raise RuntimeError(f"{self.pool.n} slots are taken and {type(self.engine).__name__} cannot grow")
             self.engine.grow(n)
             self.pool.grow(n)
         items = []

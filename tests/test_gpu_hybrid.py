@@ -509,3 +509,22 @@ def test_launch_errors(zoo):
             eng.launch(items)
     with pytest.raises(ValueError):
         m.step_engine(1, 5000)
+
+
+def test_trace_runner_serves_the_other_family(tmp_path, capsys):
+    """The same runner on a OneBit LLaMA folder: class, engine and precision chosen by config.json."""
+    import io
+    from onebit_amd.checkpoint import save_inference_checkpoint
+    from onebit_amd.llama import OneBitLlamaConfig, build_synthetic_model
+    from onebit_amd.trace import run as trace_run
+    cfg = OneBitLlamaConfig(vocab_size=96, hidden_size=128, intermediate_size=352, num_hidden_layers=2, num_attention_heads=2, max_position_embeddings=64)
+    model = build_synthetic_model(cfg, seed=1, device="cuda")
+    save_inference_checkpoint(model, str(tmp_path))
+    a, b = tokens(12, 96, 1), tokens(7, 96, 2)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:11], "want": [3, 10]}, {"id": "b", "tokens": b[:6], "want": [5]}], "end": []},
+             {"step": 1, "entries": [{"id": "a", "tokens": a[11:], "want": [0]}, {"id": "b", "tokens": b[6:], "want": []}], "end": ["a", "b"]}]
+    assert trace_run(str(tmp_path), "bfloat16", str(tmp_path / "o"), 64, lines=io.StringIO("\n".join(map(json.dumps, steps)))) == 0
+    capsys.readouterr()
+    ra, rb = (model(torch.tensor([t], device="cuda"))[0].double().cpu() for t in (a, b))
+    load = lambda i: torch.frombuffer(bytearray((tmp_path / "o" / f"{i}.f32").read_bytes()), dtype=torch.float32).view(-1, 96)
+    assert err(load(0), torch.stack([ra[3], ra[10], rb[5]])) < 0.02 and err(load(1), ra[[11]]) < 0.02
