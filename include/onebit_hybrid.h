@@ -44,7 +44,7 @@ typedef struct onebit_hlayer {
     const float *conv_w, *conv_b, *dt_bias, *A_log, *D, *gnorm_w;     /* conv_w [taps][channels]                                  */
 } onebit_hlayer_t;
 
-typedef struct onebit_hrun {     /* one pass over a layer; a looped stretch lists its layers once per pass                        */
+typedef struct onebit_hrun {     /* one pass over a layer; a repeated layer appears once per repetition                        */
     int32_t layer, add_embedding;
     void *s0, *s1;               /* attention: k [slots][kv_heads][max_len][kp], v [..][vp]; state space: fp32 state
                                     [slots][heads][state][sp], convolution ring [slots][taps][channels]                          */

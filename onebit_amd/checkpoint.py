@@ -90,8 +90,7 @@ _ST_DTYPES = {"F64": torch.float64, "F32": torch.float32, "F16": torch.float16, 
 
 
 def read_safetensors(path: str) -> Dict[str, torch.Tensor]:
-    """The tensors of a safetensors file: 8-byte little-endian header length, JSON header (name -> dtype, shape, data_offsets), data.
-    Nothing in the file is executed; offsets and sizes are checked.  The tensors are views of a private memory map."""
+    """The tensors of a safetensors file (u64 header size, JSON header, raw data).  Nothing in the file is executed; offsets and sizes are checked.  The tensors are views of a private memory map."""
     with open(path, "rb") as f:
         size = os.fstat(f.fileno()).st_size
         n = struct.unpack("<Q", f.read(8))[0] if size >= 8 else size

@@ -1,7 +1,7 @@
 """Command line: ``python -m onebit_amd <command>``.  The model class is chosen by the folder's config.json.
 
   generate   greedy continuation of token ids through the continuous batcher
-  trace      replay a trace of steps from standard input (also: bin/trace_run)"""
+  trace      replay a recorded schedule of steps (also: bin/trace_run)"""
 from __future__ import annotations
 
 import argparse
@@ -14,11 +14,11 @@ def _trace_args(ap: argparse.ArgumentParser):
     ap.add_argument("--dtype", choices=["bfloat16", "float32"], default="bfloat16",
                     help="bfloat16: the family's serving kernels; float32: everything in 32-bit (exit code 3 if the family has no such kernels)")
     ap.add_argument("--out", required=True, help="folder for the logits")
-    ap.add_argument("--max-tokens", type=int, required=True, help="the most tokens that live requests hold at any time")
+    ap.add_argument("--max-tokens", type=int, required=True, help="upper bound of the tokens held by all open requests together (sizes the cache)")
 
 
 def trace_main(argv=None) -> int:
-    ap = argparse.ArgumentParser(prog="trace_run", description="feed given token ids through a model, step by step, and write logits")
+    ap = argparse.ArgumentParser(prog="trace_run", description="replay a recorded schedule of steps through a model's serving engine and dump logits")
     _trace_args(ap)
     a = ap.parse_args(argv)
     from .trace import run

@@ -7,7 +7,7 @@ Every layer is the parallel form  x += mult * (mixer(norm(x)) + ff(norm(x)))  as
 normalised row, so their input projections are ONE weight matrix, and their output projections act on disjoint column ranges of one
 row, so they are one matrix too (csrc/ob_dense.h has the packed layout).
 
-``StateSlots`` holds what requests leave between steps, per layer RUN (a looped stretch keeps one cache or state per pass): keys and
+``StateSlots`` holds what requests leave between steps, per layer RUN (a layer that a loop repeats has an entry for each repetition): keys and
 values, or the fp32 recurrent state and the ring of convolution inputs.  ``HybridStep`` is the step engine with ``MixedStep``'s
 interface: items in, greedy tokens and logits out; single-token steps replay a HIP graph."""
 from __future__ import annotations
@@ -280,7 +280,7 @@ class HybridDecoder:
 
     @torch.no_grad()
     def generate(self, input_ids: torch.Tensor, max_new_tokens: int, eos_token_id=None, pad_token_id=None) -> torch.Tensor:
-        """Greedy search with the contract of ``OneBitLlamaForCausalLM.generate``, one batcher slot per row."""
+        """Greedy search as ``OneBitLlamaForCausalLM.generate`` (same arguments and result), one batcher slot per row."""
         from .serving import generate_batched
         return generate_batched(self, input_ids, max_new_tokens, eos_token_id, pad_token_id, self._engines)
 

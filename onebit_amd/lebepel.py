@@ -1,8 +1,8 @@
 """Lebepel: a decoder-only model of sigmoid-attention and state-space layers with parallel feed-forwards, learned positions and a looped
 stretch of layers.  This file reads its config.json and tensors and describes it with the parts of ``hybrid.py``; nothing here computes.
 
-Per layer: h = rms(x) (1 + w), x += residual_mult (mixer(h) + ff(h)).  ``loop`` runs layers start .. stop - 1 ``times`` times, each pass
-with its own cache or state; before every pass but the first the embedding output is added to x.  Logits are soft-capped."""
+Per layer: h = rms(x) (1 + w), x += residual_mult (mixer(h) + ff(h)).  ``loop`` repeats a stretch of layers: every repetition keeps state
+of its own, and from the second one on it starts by adding the embedding rows to the residual stream.  Logits are soft-capped."""
 from __future__ import annotations
 
 import json

@@ -601,7 +601,7 @@ def batched_rows(model, prompts: List[List[int]], max_new_tokens: int, max_posit
 
 @torch.no_grad()
 def generate_batched(model, input_ids: torch.Tensor, max_new_tokens: int, eos_token_id=None, pad_token_id=None, engines: Optional[Dict] = None) -> torch.Tensor:
-    """``generate``'s contract (input_ids [B, S] -> prompts followed by up to ``max_new_tokens`` greedy tokens) on the batcher."""
+    """The batched form of ``generate`` (input_ids [B, S] -> prompts followed by up to ``max_new_tokens`` greedy tokens) on the batcher."""
     if input_ids.dim() != 2:
         raise ValueError("input_ids must be [B, S]")
     if max_new_tokens < 1:

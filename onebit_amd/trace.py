@@ -1,11 +1,11 @@
-"""Replay a trace: given token ids through a model step by step, logits out.  Nothing is sampled; the steps run on the family's step
-engine over its cache / state slots, as the batcher's do.
+"""Trace replay: a recorded schedule of steps run on the family's step engine and cache / state slots exactly as the batcher runs its own,
+with logits instead of sampling.
 
-Standard input, one JSON object a line:
-  {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
-``entries``: each request's next tokens and the places among them whose logits are wanted; ``end``: requests finished after the step (their
-slots are given back).  A step in which something is wanted writes OUT/<step>.f32, little-endian fp32 [wanted, vocab] in entry order;
-after every step ``done <step>`` is printed."""
+One step per input line, as JSON:
+  {"step": 7, "entries": [{"id": "req-1", "tokens": [11, 4], "want": [1]}, {"id": "req-2", "tokens": [9], "want": []}], "end": ["req-2"]}
+An entry continues its request (or opens it) by ``tokens``; ``want`` indexes the tokens to report logits for; ``end`` frees the slots of the
+requests it names once the step has run.  Reported logits go to OUT/<step>.f32 as raw little-endian fp32 rows of ``vocab`` values, entry by
+entry; steps that report nothing write no file.  Each step is acknowledged with a line ``done <step>``."""
 from __future__ import annotations
 
 import json

@@ -12,7 +12,7 @@ def rms(x, eps):
 
 
 def norm(x, w, eps):
-    """RMS norm whose weight is stored around zero."""
+    """RMS norm with scale 1 + w."""
     return rms(x, eps) * (1 + w)
 
 
@@ -61,7 +61,7 @@ def attention(h, w, p, mix, eps):
 
 
 def short_conv(x, taps, bias):
-    """Causal convolution per channel: x [T, ch], taps [ch, n] (last column = the current token), zeros before the start."""
+    """y_t = bias + sum_j taps[:, j] x_{t - (n - 1) + j}, channel by channel; x_s = 0 for s < 0.  x [T, ch], taps [ch, n]."""
     T, n = x.shape[0], taps.shape[1]
     y = torch.zeros_like(x) + bias
     for t in range(T):
@@ -86,7 +86,7 @@ def ssm(x, B, C, dt, A_log, D):
 
 
 def gated_group_norm(y, z, w, groups, eps):
-    """y * silu(z) first, then each of ``groups`` equal parts by its own root mean square, times w."""
+    """v = y silu(z); rms over each of ``groups`` slices of v, scaled by w."""
     T = y.shape[0]
     return rms((y * silu(z)).view(T, groups, -1), eps).reshape(T, -1) * w
 
