@@ -72,8 +72,8 @@ SYMBOLS = {
 
 # libonebit_hybrid.so (include/onebit_hybrid.h): the hybrid decoders
 HYBRID_LIB_PATH = os.path.join(_HERE, "csrc", "libonebit_hybrid.so")
-HYBRID_ABI_VERSION = 1
-HYB_BF16, HYB_F32 = 2, 1
+HYBRID_ABI_VERSION = 2
+HYB_BF16, HYB_F32, HYB_SHORT = 2, 1, 16
 HYBRID_SYMBOLS = {
     "onebit_hybrid_abi_version": (_int, []),
     "onebit_hybrid_last_error": (ctypes.c_char_p, []),

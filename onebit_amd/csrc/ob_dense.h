@@ -71,6 +71,21 @@ template <typename E> __device__ __forceinline__ float ob_silu(float z)
 {
     if constexpr (sizeof(E) == 2) return ob_silu_fast(z); else return ob_siluf(z);
 }
+// tanh form of gelu; 0.5 (1 + tanh(u)) = sigmoid(2 u)
+template <typename E> __device__ __forceinline__ float ob_gelu_tanh(float z)
+{
+    const float u = 0.79788456080286536f * (z + 0.044715f * z * z * z);
+    if constexpr (sizeof(E) == 2) return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-2.8853900817779268f * u));
+    else return 0.5f * z * (1.0f + tanhf(u));
+}
+// quadratic above zero, exponential below, slope 1/2 at zero:  a z^2 + z / 2  |  b (e^z - 1 - z) + z / 2
+template <typename E> __device__ __forceinline__ float ob_xielu(float z, float a, float b)
+{
+    const float n = fminf(z, 0.f);
+    float em;
+    if constexpr (sizeof(E) == 2) em = __builtin_amdgcn_exp2f(1.4426950408889634f * n) - 1.0f; else em = expm1f(n);
+    return z > 0.f ? __builtin_fmaf(a * z, z, 0.5f * z) : __builtin_fmaf(b, em - n, 0.5f * z);
+}
 __device__ __forceinline__ float ob_softplusf(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
 
 // ---- what a product's output becomes -------------------------------------------------------------------------------------
@@ -79,7 +94,20 @@ __device__ __forceinline__ float ob_softplusf(float z) { return fmaxf(z, 0.0f) +
 //                 fragment-major rows of the output product, at column act_k0
 //   OB_EPI_PART   fp32 partial sums z[split][t][n] (the layer's output product: the row kernel that follows adds the splits)
 //   OB_EPI_LOGITS fp32 logits[t][n], cap * tanh(v / cap) when cap > 0
-enum { OB_EPI_IN = 0, OB_EPI_PART = 1, OB_EPI_LOGITS = 2 };
+//   OB_EPI_ACT    f(v) into fragment-major rows at column act_k0 + n: f = identity, xIELU, or gelu_tanh(v) times an entry of the token's row
+//                 of a table
+//   OB_EPI_HEADS  head-major rows: heads[n / D][t][n % D] (D a power of two), keys and values of a prompt's latents
+enum ObEpilogue { OB_EPI_IN = 0, OB_EPI_PART = 1, OB_EPI_LOGITS = 2, OB_EPI_ACT = 3, OB_EPI_HEADS = 4 };
+enum ObDenseFn { OB_FN_ID = 0, OB_FN_XIELU = 1, OB_FN_GELU_TABLE = 2 };
+
+// ---- which weights meet which rows ------------------------------------------------------------------------------------------
+//   OB_ROWS_ALL     every row, fragment-major activations
+//   OB_ROWS_HEADS   block-diagonal over heads: n tiles tile_group apart read their own act_cols columns of ROW-MAJOR activations
+//   OB_ROWS_GATHER  blocks of one expert's rows (ObRowBlock table): activation row gather[row] of a ROW-MAJOR matrix, output row `row`
+//   OB_ROWS_SORTED  the same blocks, fragment-major activations in block order
+//   OB_ROWS_SEGS    rows of several requests' cache slots (fragment-major bands), output rows consecutive per request
+enum ObRowForm { OB_ROWS_ALL = 0, OB_ROWS_HEADS = 1, OB_ROWS_GATHER = 2, OB_ROWS_SORTED = 3, OB_ROWS_SEGS = 4 };
+struct ObRowBlock { int32_t group, row0, count, pad; };      // rows [row0, row0 + count) of weight group `group`; row0 a multiple of 16 at a group's start
 
 struct ObDenseArgs {
     const void *w, *a;             // fragment-major weights [n_tiles][nkt], activations [t tiles][nkt]
@@ -94,14 +122,54 @@ struct ObDenseArgs {
     float *z; int ldz; size_t z_split;
     // OB_EPI_LOGITS
     float *logits; int V; float cap;
+    // OB_EPI_ACT (act, act_k0, act_nkt as above)
+    int fn; float fa, fb;          // xIELU's two factors
+    const void *table; const int32_t *tokens; int ld_table, table_cols;      // entry (tokens[t], n), n < table_cols
+    // OB_EPI_HEADS
+    void *heads; int d_shift, head_rows;
+    // OB_ROWS_HEADS / OB_ROWS_GATHER: row-major activations
+    int lda, tile_group, act_cols;
+    // OB_ROWS_GATHER / OB_ROWS_SORTED
+    const ObRowBlock *blk; const int32_t *gather; size_t w_group;             // weight tiles per group
 };
+#define OB_DENSE_MAXSEG 64
+struct ObDenseSegArgs : ObDenseArgs {          // OB_ROWS_SEGS: token block b belongs to segment i with blk_end[i - 1] <= b < blk_end[i]
+    int nseg;
+    int blk_end[OB_DENSE_MAXSEG];
+    int band0[OB_DENSE_MAXSEG], row0[OB_DENSE_MAXSEG], rows[OB_DENSE_MAXSEG];
+};
+
+// (a class template, not an expression of the row form: kernel names must be the same on host and device)
+template <int ROWS> struct ObDenseArgsOf { typedef ObDenseArgs type; };
+template <> struct ObDenseArgsOf<OB_ROWS_SEGS> { typedef ObDenseSegArgs type; };
 
 // one n-tile pair (nt even) of one token tile: lane = (token t, columns 16 nt + 4 g ..), (token t, columns 16 (nt + 1) + 4 g ..)
 template <typename E, int EPI>
-__device__ __forceinline__ void ob_dense_epilogue(const ObDenseArgs &A, int nt, int t, int g, ob_float4 v0, ob_float4 v1, int split)
+__device__ __forceinline__ void ob_dense_epilogue(const ObDenseArgs &A, int nt, int t, bool live, int g, ob_float4 v0, ob_float4 v1, int split)
 {
-    if (t >= A.T) return;
-    if constexpr (EPI == OB_EPI_PART) {
+    if (!live) return;
+    if constexpr (EPI == OB_EPI_ACT || EPI == OB_EPI_HEADS) {
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+            if (nt + h >= A.n_tiles) return;
+            ob_float4 v = h ? v1 : v0;
+            const int n = (nt + h) * 16 + 4 * g;
+            if constexpr (EPI == OB_EPI_HEADS) {
+                const int hd = n >> A.d_shift, d = n & ((1 << A.d_shift) - 1);
+                *reinterpret_cast<typename ObElem<E>::V4 *>((E *)A.heads + ((((size_t)hd * A.head_rows + t) << A.d_shift) + d)) = ob_to_v4<E>(v);
+            } else {
+                if (A.fn == OB_FN_XIELU) {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) v[e] = ob_xielu<E>(v[e], A.fa, A.fb);
+                } else if (A.fn == OB_FN_GELU_TABLE) {
+                    const E *row = (const E *)A.table + (size_t)A.tokens[t] * A.ld_table;
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) v[e] = n + e < A.table_cols ? ob_gelu_tanh<E>(v[e]) * (float)row[n + e] : 0.f;
+                }
+                *reinterpret_cast<typename ObElem<E>::V4 *>((E *)A.act + ob_frag<E>(t, A.act_k0 + n, A.act_nkt)) = ob_to_v4<E>(v);
+            }
+        }
+    } else if constexpr (EPI == OB_EPI_PART) {
         float *z = A.z + (size_t)split * A.z_split + (size_t)t * A.ldz;
         if (nt < A.n_tiles) *reinterpret_cast<ob_float4 *>(z + nt * 16 + 4 * g) = v0;
         if (nt + 1 < A.n_tiles) *reinterpret_cast<ob_float4 *>(z + nt * 16 + 16 + 4 * g) = v1;
@@ -150,7 +218,9 @@ __device__ __forceinline__ void ob_dense_epilogue(const ObDenseArgs &A, int nt, 
 // Workgroup = 2 n tiles (32 output columns; a gate / up pair) x all token tiles x one K split; its four waves take a quarter of the
 // split's k tiles each and add up through LDS.  Activations come from L2 (1 KB linear loads).  The next U k tiles are requested
 // before the current U are multiplied: U * 2 KB of weights per wave in flight.
-template <typename E, int EPI, int MT>
+// Row-major activations (OB_ROWS_HEADS, OB_ROWS_GATHER): a lane's 16 bytes come from its own row, 64 bytes per row and k tile.
+// Expert blocks: grid.z = entries of the block table (count 0: nothing to do).
+template <typename E, int EPI, int MT, int ROWS = OB_ROWS_ALL>
 __global__ __launch_bounds__(256, MT >= 4 ? 2 : 3) void ob_dense_skinny_kernel(const ObDenseArgs A)
 {
     typedef typename ObElem<E>::V16 V16;
@@ -161,9 +231,26 @@ __global__ __launch_bounds__(256, MT >= 4 ? 2 : 3) void ob_dense_skinny_kernel(c
     const int k_lo = split * A.kt_split, k_hi = min(A.nkt, k_lo + A.kt_split);
     const int per = (k_hi - k_lo + 3) >> 2;
     const int k0 = k_lo + wave * per, k1 = min(k0 + per, k_hi);
-    const V16 *w0 = (const V16 *)A.w + (size_t)nt * A.nkt * 64 + lane;
-    const V16 *w1 = (const V16 *)A.w + (size_t)min(nt + 1, A.n_tiles - 1) * A.nkt * 64 + lane;
-    const V16 *ap = (const V16 *)A.a + lane;
+    int t0 = 0, rows = A.T;
+    size_t wg = 0;
+    if constexpr (ROWS == OB_ROWS_GATHER || ROWS == OB_ROWS_SORTED) {
+        const ObRowBlock b = A.blk[blockIdx.z];
+        if (b.count <= 0) return;                        // (uniform)
+        t0 = b.row0; rows = b.count; wg = (size_t)b.group * A.w_group;
+    }
+    const V16 *w0 = (const V16 *)A.w + (wg + (size_t)nt * A.nkt) * 64 + lane;
+    const V16 *w1 = (const V16 *)A.w + (wg + (size_t)min(nt + 1, A.n_tiles - 1) * A.nkt) * 64 + lane;
+    // this lane's piece of k tile 0 of every token tile, and the step (in 16 bytes) to the next k tile
+    const V16 *ap[MT];
+    constexpr int KSTEP = ROWS == OB_ROWS_HEADS || ROWS == OB_ROWS_GATHER ? 4 : 64;
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+        if constexpr (ROWS == OB_ROWS_HEADS)
+            ap[m] = (const V16 *)((const E *)A.a + (size_t)min(m * 16 + (lane & 15), rows - 1) * A.lda + nt / A.tile_group * A.act_cols) + (lane >> 4);
+        else if constexpr (ROWS == OB_ROWS_GATHER)
+            ap[m] = (const V16 *)((const E *)A.a + (size_t)A.gather[t0 + min(m * 16 + (lane & 15), rows - 1)] * A.lda) + (lane >> 4);
+        else ap[m] = (const V16 *)A.a + lane + (size_t)((t0 >> 4) + m) * A.nkt * 64;
+    }
     ob_float4 acc[2][MT];
 #pragma unroll
     for (int m = 0; m < MT; ++m) acc[0][m] = acc[1][m] = (ob_float4){0.f, 0.f, 0.f, 0.f};
@@ -175,7 +262,7 @@ __global__ __launch_bounds__(256, MT >= 4 ? 2 : 3) void ob_dense_skinny_kernel(c
             wd[0][u] = __builtin_nontemporal_load(w0 + (size_t)kk * 64);
             wd[1][u] = __builtin_nontemporal_load(w1 + (size_t)kk * 64);
 #pragma unroll
-            for (int m = 0; m < MT; ++m) ad[m][u] = ap[((size_t)m * A.nkt + kk) * 64];
+            for (int m = 0; m < MT; ++m) ad[m][u] = ap[m][(size_t)kk * KSTEP];
         }
     };
     if (k0 < k1) {                                       // (wave-uniform)
@@ -212,7 +299,8 @@ __global__ __launch_bounds__(256, MT >= 4 ? 2 : 3) void ob_dense_skinny_kernel(c
         ob_float4 v[2];
 #pragma unroll
         for (int h = 0; h < 2; ++h) v[h] = (red[0][h][m][lane] + red[1][h][m][lane]) + (red[2][h][m][lane] + red[3][h][m][lane]);
-        ob_dense_epilogue<E, EPI>(A, nt, m * 16 + (lane & 15), lane >> 4, v[0], v[1], split);
+        const int tl = m * 16 + (lane & 15);
+        ob_dense_epilogue<E, EPI>(A, nt, t0 + tl, tl < rows, lane >> 4, v[0], v[1], split);
     }
 }
 
@@ -227,9 +315,10 @@ __device__ __forceinline__ void ob_dma_1k(const char *base, uint32_t lane_off, u
                  : "=&s"(keep) : "s"(lds_addr), "v"(lane_off), "s"(base) : "memory");
 }
 
-template <typename E, int EPI, int NB, int TB, int WN, int WT, int NST>
-__global__ __launch_bounds__(64 * WN * WT, 2) void ob_dense_tile_kernel(const ObDenseArgs A)
+template <typename E, int EPI, int NB, int TB, int WN, int WT, int NST, int ROWS = OB_ROWS_ALL>
+__global__ __launch_bounds__(64 * WN * WT, 2) void ob_dense_tile_kernel(const typename ObDenseArgsOf<ROWS>::type A)
 {
+    static_assert(ROWS != OB_ROWS_HEADS, "the block-diagonal form has few rows only");
     typedef typename ObElem<E>::V16 V16;
     constexpr int NW = WN * WT, TILES = NB + TB, PER = TILES / NW, MN = NB / WN, MT = TB / WT;
     static_assert(TILES % NW == 0 && NB % WN == 0 && TB % WT == 0 && MN % 2 == 0, "tile shape");
@@ -238,26 +327,50 @@ __global__ __launch_bounds__(64 * WN * WT, 2) void ob_dense_tile_kernel(const Ob
     const int wn = wave % WN, wt = wave / WN;
     // XCD-aware numbering: workgroup ids are dealt round-robin to the 8 XCDs; give each a contiguous range of logical tiles, token
     // blocks fastest, so that the tiles in flight on an XCD share weight bands and activation rows in its L2
-    const int ntb = (A.T + TB * 16 - 1) / (TB * 16);
+    const int ntb = (A.T + TB * 16 - 1) / (TB * 16);                   // (grouped forms: T = 16 TB times the number of blocks)
     const int nwg = gridDim.x, orig = blockIdx.x, xcd = orig & 7, q8 = nwg >> 3, rem = nwg & 7;
     const int bid = (xcd < rem ? xcd * (q8 + 1) : rem * (q8 + 1) + (xcd - rem) * q8) + (orig >> 3);
     const int nb = bid / ntb, tb = bid - nb * ntb;
-    const int n0 = nb * NB, t0 = tb * TB, split = blockIdx.y;
+    const int n0 = nb * NB, split = blockIdx.y;
+    // rows of this block: `rows` of them, activations from band `band0` on, outputs from row `out0` on
+    int band0 = tb * TB, out0 = tb * TB * 16, rows = A.T - out0;
+    size_t wg = 0;
+    if constexpr (ROWS == OB_ROWS_GATHER || ROWS == OB_ROWS_SORTED) {
+        const ObRowBlock b = A.blk[tb];
+        if (b.count <= 0) return;                                     // (uniform)
+        band0 = b.row0 >> 4; out0 = b.row0; rows = b.count; wg = (size_t)b.group * A.w_group;
+    } else if constexpr (ROWS == OB_ROWS_SEGS) {
+        int sg = 0;
+        while (sg < A.nseg - 1 && tb >= A.blk_end[sg]) ++sg;
+        const int loc = (tb - (sg ? A.blk_end[sg - 1] : 0)) * TB;
+        band0 = A.band0[sg] + loc; out0 = A.row0[sg] + loc * 16; rows = A.rows[sg] - loc * 16;
+    }
     const int k_lo = split * A.kt_split, k_hi = min(A.nkt, k_lo + A.kt_split), nk = k_hi - k_lo;
-    const int t_tiles = (A.T + 15) >> 4;
+    const int t_tiles = (rows + 15) >> 4;
     const char *src[PER];
+    uint32_t loff[PER], kstep[PER];                                   // (two values, wave-uniform step: 1 KB tiles, or 64 bytes of a gathered row)
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
         const int j = wave * PER + i;
-        const size_t band = j < NB ? (size_t)min(n0 + j, A.n_tiles - 1) : (size_t)min(t0 + j - NB, t_tiles - 1);
-        src[i] = (const char *)(j < NB ? A.w : A.a) + (band * A.nkt + k_lo) * 1024;
+        const size_t band = j < NB ? (size_t)min(n0 + j, A.n_tiles - 1) : (size_t)(band0 + min(j - NB, t_tiles - 1));
+        src[i] = (const char *)(j < NB ? A.w : A.a) + ((j < NB ? wg : 0) + band * A.nkt + k_lo) * 1024;
+        loff[i] = lane * 16;
+        kstep[i] = 1024;
+        if constexpr (ROWS == OB_ROWS_GATHER) {
+            if (j >= NB) {
+                src[i] = (const char *)A.a + (size_t)k_lo * 64;
+                loff[i] = (uint32_t)A.gather[out0 + min((j - NB) * 16 + (lane & 15), rows - 1)] * (uint32_t)(A.lda * sizeof(E)) + (lane >> 4) * 16;
+                kstep[i] = 64;
+            }
+        }
     }
     const uint32_t lds0 = (uint32_t)(size_t)(__attribute__((address_space(3))) char *)smem;
-    const uint32_t lane_off = lane * 16;
     auto dma = [&](int k, int buf) {
-        const size_t ko = (size_t)min(k, nk - 1) * 1024;
+        const size_t kk = (size_t)min(k, nk - 1);
 #pragma unroll
-        for (int i = 0; i < PER; ++i) ob_dma_1k(src[i] + ko, lane_off, lds0 + (uint32_t)(buf * TILES + wave * PER + i) * 1024);
+        for (int i = 0; i < PER; ++i)
+            ob_dma_1k(src[i] + kk * (ROWS == OB_ROWS_GATHER ? kstep[i] : 1024), ROWS == OB_ROWS_GATHER ? loff[i] : lane * 16,
+                      lds0 + (uint32_t)(buf * TILES + wave * PER + i) * 1024);
     };
     ob_float4 acc[MN][MT];
 #pragma unroll
@@ -288,8 +401,8 @@ __global__ __launch_bounds__(64 * WN * WT, 2) void ob_dense_tile_kernel(const Ob
     const int g = lane >> 4;
 #pragma unroll
     for (int j = 0; j < MT; ++j) {
-        const int t = (t0 + wt * MT + j) * 16 + (lane & 15);
+        const int tl = (wt * MT + j) * 16 + (lane & 15);
 #pragma unroll
-        for (int i = 0; i < MN; i += 2) ob_dense_epilogue<E, EPI>(A, n0 + wn * MN + i, t, g, acc[i][j], acc[i + 1][j], split);
+        for (int i = 0; i < MN; i += 2) ob_dense_epilogue<E, EPI>(A, n0 + wn * MN + i, out0 + tl, tl < rows, g, acc[i][j], acc[i + 1][j], split);
     }
 }

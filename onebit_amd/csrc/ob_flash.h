@@ -73,8 +73,10 @@ struct ObFlashRaggedArgs {
     ObFlashSeg seg[OB_FL_MAXSEG];
 };
 
-// How scores become weights.  The kernel below is written once for both:
+// How scores become weights.  The kernel below is written once for all:
 //   ObFlSoftmaxF16   fp16 operands, online softmax (the OneBit LLaMA attention)
+//   ObFlSoftmaxBf16  bf16 operands, online softmax; keys and values head-major [Hkv][max_len][D] with a segment's keys from row `slot` on (the
+//                    rows a latent cache was expanded to); weights as two bf16 terms like the sigmoid form's; fragment-major output
 //   ObFlSigmoidBf16  bf16 operands, w = 1 / (1 + 2^a), a = q.k (-scale log2 e) + (r1 log2(1 + r2 distance) - pb log2 e), not normalised:
 //                    no maxima, no sums, no rescale.  The distance term of a block depends on query - key only (191 values per
 //                    128 x 64 block): a table in LDS, written beside the block's K / V tiles.  The weights enter the value product as two
@@ -82,7 +84,7 @@ struct ObFlashRaggedArgs {
 struct ObFlSoftmaxF16 {
     typedef _Float16 H;
     typedef ob_half8 V8;
-    static constexpr bool SOFTMAX = true;
+    static constexpr bool SOFTMAX = true, BF16 = false, HEAD_MAJOR = false;      // (BF16: weights enter the value product as hi + lo)
     static __device__ __forceinline__ ob_float4 mfma(V8 a, V8 b, ob_float4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_f16(a, b, c, 0, 0, 0); }
     typedef ObFlashRaggedArgs RaggedArgs;
 };
@@ -96,12 +98,15 @@ struct ObFlashSigArgs : ObFlashRaggedArgs {      // a.q [rows, H, D], a.k / a.v 
 struct ObFlSigmoidBf16 {
     typedef __bf16 H;
     typedef ob_u32x4 V8;              // (operands kept as dwords: hipcc takes vectors of __bf16 apart and spills)
-    static constexpr bool SOFTMAX = false;
+    static constexpr bool SOFTMAX = false, BF16 = true, HEAD_MAJOR = false;
     static __device__ __forceinline__ ob_float4 mfma(V8 a, V8 b, ob_float4 c)
     {
         return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(ob_fl_bf8, a), __builtin_bit_cast(ob_fl_bf8, b), c, 0, 0, 0);
     }
     typedef ObFlashSigArgs RaggedArgs;
+};
+struct ObFlSoftmaxBf16 : ObFlSigmoidBf16 {
+    static constexpr bool SOFTMAX = true, HEAD_MAJOR = true;
 };
 
 #define OB_FL_BM 128
@@ -143,7 +148,8 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
     typedef typename POL::H H16;
     typedef typename POL::V8 V8;
     constexpr bool SM = POL::SOFTMAX;
-    static_assert(SM || RAGGED, "the sigmoid form has ragged rows only");
+    constexpr bool B16 = POL::BF16;
+    static_assert(!B16 || RAGGED, "the bf16 forms have ragged rows only");
     const ObFlashArgs &A = [&]() -> const ObFlashArgs & { if constexpr (RAGGED) return AA.a; else return AA; }();
     constexpr int DT = D / 16, DK = D / 32;
     constexpr int NPC = D / 8;                  // 16-byte pieces per K / V row
@@ -196,8 +202,9 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
     const int L = past + S;
     // K / V rows of this head as buffer resources: the offset of a piece is (lane-constant) + (block-uniform scalar), no per-block
     // address arithmetic, and rows beyond the last key read as zeros (they are masked; zeros keep 0 x V finite)
-    const __amdgpu_buffer_rsrc_t krs = __builtin_amdgcn_make_buffer_rsrc((void *)(A.k + ((int64_t)b * A.Hkv + kvh) * A.max_len * D), 0, L * D * 2, 0x00020000);
-    const __amdgpu_buffer_rsrc_t vrs = __builtin_amdgcn_make_buffer_rsrc((void *)(A.v + ((int64_t)b * A.Hkv + kvh) * A.max_len * D), 0, L * D * 2, 0x00020000);
+    const int64_t kv_off = POL::HEAD_MAJOR ? ((int64_t)kvh * A.max_len + b) * D : ((int64_t)b * A.Hkv + kvh) * A.max_len * D;
+    const __amdgpu_buffer_rsrc_t krs = __builtin_amdgcn_make_buffer_rsrc((void *)(A.k + kv_off), 0, L * D * 2, 0x00020000);
+    const __amdgpu_buffer_rsrc_t vrs = __builtin_amdgcn_make_buffer_rsrc((void *)(A.v + kv_off), 0, L * D * 2, 0x00020000);
 
     float dist_r1 = 0.f, dist_r2 = 0.f, dist_pb = 0.f;
     if constexpr (!SM) {
@@ -433,16 +440,46 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
                     }
                 l_run[qt] += ls;
                 // P^T operands: k-elements of step ks = this lane's 4 keys of tile 2 ks, then of tile 2 ks + 1
+                if constexpr (!B16) {
 #pragma unroll
-                for (int ks = 0; ks < 2; ++ks)
+                    for (int ks = 0; ks < 2; ++ks)
 #pragma unroll
-                    for (int e = 0; e < 4; ++e) {
-                        pb[qt][ks][e] = (_Float16)sc[2 * ks][qt][e];
-                        pb[qt][ks][4 + e] = (_Float16)sc[2 * ks + 1][qt][e];
-                    }
+                        for (int e = 0; e < 4; ++e) {
+                            pb[qt][ks][e] = (_Float16)sc[2 * ks][qt][e];
+                            pb[qt][ks][4 + e] = (_Float16)sc[2 * ks + 1][qt][e];
+                        }
+                }
             }
 #endif
             OB_FL_T(3);
+            if constexpr (B16) {
+                // 32 keys at a time, weights as hi + lo (as the sigmoid form)
+#pragma unroll
+                for (int ks = 0; ks < 2; ++ks) {
+                    ob_u32x4 wh[2], wl[2];
+                    if (ks == 1) {
+                        if (D > 64) __builtin_amdgcn_sched_barrier(0);
+                        read_v(1);
+                    }
+#pragma unroll
+                    for (int qt = 0; qt < 2; ++qt)
+#pragma unroll
+                        for (int i2 = 0; i2 < 4; ++i2) {
+                            const float w0 = sc[2 * ks + (i2 >> 1)][qt][2 * (i2 & 1)], w1 = sc[2 * ks + (i2 >> 1)][qt][2 * (i2 & 1) + 1];
+                            const float r0 = w0 - __uint_as_float(__float_as_uint(w0) & 0xffff0000u), r1 = w1 - __uint_as_float(__float_as_uint(w1) & 0xffff0000u);
+                            wh[qt][i2] = __builtin_amdgcn_perm(__float_as_uint(w1), __float_as_uint(w0), 0x07060302u);
+                            wl[qt][i2] = __builtin_bit_cast(uint32_t, __builtin_convertvector((ob_float2){r0, r1}, ob_fl_bf2));
+                        }
+                    if (D > 64) __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+                    for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+                        for (int qt = 0; qt < 2; ++qt) {
+                            acc_o[dt][qt] = POL::mfma(vf[ks][dt], __builtin_bit_cast(V8, wh[qt]), acc_o[dt][qt]);
+                            acc_o[dt][qt] = POL::mfma(vf[ks][dt], __builtin_bit_cast(V8, wl[qt]), acc_o[dt][qt]);
+                        }
+                }
+            } else {
             // ---- O^T += V^T . P^T
             read_v(1);
             __builtin_amdgcn_sched_barrier(0);
@@ -452,6 +489,7 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
                 for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
                     for (int qt = 0; qt < 2; ++qt) acc_o[dt][qt] = POL::mfma(vf[ks][dt], pb[qt][ks], acc_o[dt][qt]);
+            }
             }
         }
         OB_FL_T(4);
@@ -473,7 +511,12 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
 #pragma unroll
     for (int qt = 0; qt < 2; ++qt) {
         const int s = m0 + 32 * wave + 16 * qt + lr;
-        if constexpr (!SM) {
+        if constexpr (B16) {
+            float inv = 1.f;
+            if constexpr (SM) {
+                const float l = ob_fl_col_sum(l_run[qt]);
+                inv = l > 0.f ? 1.0f / l : 0.f;
+            }
             if (s >= S) continue;
             const int row = (int)qrow0 + s;
             int c0 = head * AA.vdim + 4 * g;             // (opaque: the columns' offsets are formed here, not kept through the key loop)
@@ -486,13 +529,13 @@ __global__ __launch_bounds__(256, 2) void ob_flash_fwd_kernel(const std::conditi
                     if (d < AA.vdim) {
                         ob_fl_bf4 ov;
 #pragma unroll
-                        for (int e = 0; e < 4; ++e) ov[e] = (H16)acc_o[dt][qt][e];
+                        for (int e = 0; e < 4; ++e) ov[e] = (H16)(SM ? acc_o[dt][qt][e] * inv : acc_o[dt][qt][e]);
                         *reinterpret_cast<ob_fl_bf4 *>(o + (c >> 5) * 512 + ((c & 31) >> 3) * 128 + (c & 7)) = ov;
                     }
                 } else {
 #pragma unroll
                     for (int e = 0; e < 4; ++e)
-                        if (d + e < AA.vdim) o[((c + e) >> 5) * 512 + (((c + e) & 31) >> 3) * 128 + ((c + e) & 7)] = (H16)acc_o[dt][qt][e];
+                        if (d + e < AA.vdim) o[((c + e) >> 5) * 512 + (((c + e) & 31) >> 3) * 128 + ((c + e) & 7)] = (H16)(SM ? acc_o[dt][qt][e] * inv : acc_o[dt][qt][e]);
                 }
             }
             continue;

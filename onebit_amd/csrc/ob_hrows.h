@@ -86,6 +86,167 @@ __global__ __launch_bounds__(1024) void ob_hnorm_kernel(const ObHNormArgs A)
     }
 }
 
+// The same row with everything a sequential layer adds to it:
+//   s = sum of the splits (+ bias) + sum_k tok_w[k] ez[tok_row[k]] (experts) + id_w h (identity experts; h = idh or the residual itself)
+//   r = x + mult * (post_w ? s / sqrt(mean s^2 + eps) * post_w : s) (+ emb_add)
+//     or, embed != NULL: r = embed[token] * embed_scale (+ bigram[row of (previous token, token)]) (+ pos_embed[position])
+//   hist: X_i = r is kept (i = hist_i), and with dwa the stream goes on as sum_j dwa[j] X_j, j = 0 .. hist_i
+//   output: r / sqrt(mean r^2 + eps) * (off + w), or r itself (w == NULL); fragment-major and, out_rm, also row-major
+// The previous token of an item's first row comes from tok_hist [slots][max_len], where every row leaves its token.
+struct ObXRowArgs : ObHNormArgs {
+    float embed_scale; const void *bigram; int buckets, mul_prev, mul_cur;
+    int32_t *tok_hist; const int32_t *row_slot, *row_off; int n_slots, max_len;
+    const float *post_w;
+    const float *ez; size_t ez_split; int ez_n, ld_ez, top; const int32_t *tok_row; const float *tok_w, *id_w; const void *idh; int ld_idh;
+    float *hist; size_t hist_stride; int hist_i; const float *dwa;
+    void *out_rm; int ld_rm;
+};
+template <typename E, int VEC>
+__device__ __forceinline__ void ob_sum_splits(float (&s)[VEC], const float *p, size_t stride, int n)
+{
+    for (int k = 0; k < n; k += 4) {                                  // four splits in flight, added in order
+        float zv[4][VEC];
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) zv[j][e] = p[(size_t)min(k + j, n - 1) * stride + e];
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+            if (k + j < n) {
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) s[e] += zv[j][e];
+            }
+    }
+}
+template <typename E, int VEC>
+__global__ __launch_bounds__(1024) void ob_xrow_kernel(const ObXRowArgs A)
+{
+    extern __shared__ __attribute__((aligned(16))) float sm[];        // [W] row | [16] reduction
+    float *red = sm + ((A.W + 3) & ~3);
+    const int t = blockIdx.x, tid = threadIdx.x, stride = blockDim.x * VEC;
+    const int src = A.rows ? A.rows[t] : t;
+    float *xr = A.x + (size_t)src * A.W;
+    const E *er = nullptr, *pr = nullptr, *br = nullptr;
+    if (A.embed) {
+        const int tok = A.tokens[src], pos = A.row_pos[src], slot = A.row_slot[src];
+        er = (const E *)A.embed + (size_t)tok * A.W;
+        if (A.pos_embed) pr = (const E *)A.pos_embed + (size_t)max(pos, 0) * A.W;
+        if (A.bigram) {
+            const bool live = slot >= 0 && slot < A.n_slots && pos >= 0 && pos < A.max_len;
+            int b = A.buckets;                                        // (a sequence's first token)
+            if (live && pos > 0) {
+                const int prev = A.row_off[src] > 0 ? A.tokens[src - 1] : A.tok_hist[(size_t)slot * A.max_len + pos - 1];
+                b = (int)(((long long)prev * A.mul_prev + (long long)tok * A.mul_cur) % A.buckets);
+            }
+            br = (const E *)A.bigram + (size_t)b * A.W;
+            if (live && tid == 0 && !A.rows) A.tok_hist[(size_t)slot * A.max_len + pos] = tok;
+        }
+    }
+    float ss = 0.f;
+    if (!er) {
+        for (int c = tid * VEC; c < A.W; c += stride) {
+            float s[VEC];
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) s[e] = 0.f;
+            if (A.z) ob_sum_splits<E, VEC>(s, A.z + (size_t)src * A.ldz + c, A.z_split, A.n_split);
+            if (A.bias) {
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) s[e] += A.bias[c + e];
+            }
+            if (A.ez) {
+                for (int k = 0; k < A.top; ++k) {
+                    const int row = A.tok_row[(size_t)src * A.top + k];                    // (uniform)
+                    if (row < 0) continue;
+                    const float w = A.tok_w[(size_t)src * A.top + k];
+                    float y[VEC];
+#pragma unroll
+                    for (int e = 0; e < VEC; ++e) y[e] = 0.f;
+                    ob_sum_splits<E, VEC>(y, A.ez + (size_t)row * A.ld_ez + c, A.ez_split, A.ez_n);
+#pragma unroll
+                    for (int e = 0; e < VEC; ++e) s[e] = __builtin_fmaf(w, y[e], s[e]);
+                }
+            }
+            if (A.id_w) {
+                const float w = A.id_w[src];
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) s[e] = __builtin_fmaf(w, A.idh ? (float)((const E *)A.idh)[(size_t)src * A.ld_idh + c + e] : xr[c + e], s[e]);
+            }
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) { sm[c + e] = s[e]; ss = __builtin_fmaf(s[e], s[e], ss); }
+        }
+    }
+    float rp = 1.f;
+    if (A.post_w) rp = 1.0f / sqrtf(ob_block_sum(ss, red) / (float)A.W + A.eps);          // (uniform)
+    ss = 0.f;
+    for (int c = tid * VEC; c < A.W; c += stride) {
+        float r[VEC];
+        if (er) {
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) r[e] = (float)er[c + e] * A.embed_scale + (br ? (float)br[c + e] : 0.f) + (pr ? (float)pr[c + e] : 0.f);
+        } else {
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) r[e] = xr[c + e] + A.mult * (A.post_w ? sm[c + e] * rp * A.post_w[c + e] : sm[c + e]);
+            if (A.emb_add) {
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) r[e] += A.emb_add[(size_t)src * A.W + c + e];
+            }
+        }
+        if (A.hist) {
+            float *hr = A.hist + (size_t)src * A.W + c;
+            if (!A.rows) {
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) hr[A.hist_i * A.hist_stride + e] = r[e];
+            }
+            if (A.dwa) {
+                float a[VEC];
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) a[e] = 0.f;
+                for (int j = 0; j < A.hist_i; j += 4) {
+                    float v[4][VEC];
+#pragma unroll
+                    for (int q = 0; q < 4; ++q)
+#pragma unroll
+                        for (int e = 0; e < VEC; ++e) v[q][e] = hr[min(j + q, A.hist_i - 1) * A.hist_stride + e];
+#pragma unroll
+                    for (int q = 0; q < 4; ++q)
+                        if (j + q < A.hist_i) {
+#pragma unroll
+                            for (int e = 0; e < VEC; ++e) a[e] = __builtin_fmaf(A.dwa[j + q], v[q][e], a[e]);
+                        }
+                }
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) r[e] = __builtin_fmaf(A.dwa[A.hist_i], r[e], a[e]);
+            }
+        }
+        if (!A.rows) {
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) xr[c + e] = r[e];
+        }
+        if (A.emb_save) {
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) A.emb_save[(size_t)src * A.W + c + e] = r[e];
+        }
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) { sm[c + e] = r[e]; ss = __builtin_fmaf(r[e], r[e], ss); }
+    }
+    float rs = 1.f;
+    if (A.w) rs = 1.0f / sqrtf(ob_block_sum(ss, red) / (float)A.W + A.eps);               // (uniform)
+    E *out = (E *)A.out;
+    for (int c = tid * VEC; c < A.W; c += stride) {
+        ob_float4 v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) v[e] = A.w ? sm[c + e] * rs * (A.off + A.w[c + e]) : sm[c + e];
+        if constexpr (VEC == 4) {
+            const typename ObElem<E>::V4 o = ob_to_v4<E>(v);
+            *reinterpret_cast<typename ObElem<E>::V4 *>(out + ob_frag<E>(t, c, A.out_nkt)) = o;
+            if (A.out_rm) *reinterpret_cast<typename ObElem<E>::V4 *>((E *)A.out_rm + (size_t)t * A.ld_rm + c) = o;
+        } else {
+            out[ob_frag<E>(t, c, A.out_nkt)] = (E)v[0];
+            if (A.out_rm) ((E *)A.out_rm)[(size_t)t * A.ld_rm + c] = (E)v[0];
+        }
+    }
+}
+
 // grid (norm groups, rows): v = y * silu(gate); out[k0 + i] = v / sqrt(mean over the group v^2 + eps) * w
 struct ObGatedNormArgs {
     const void *y; int ldy; const void *gate; int ldg;       // row-major; the gate is the leading columns of the input product

@@ -556,17 +556,18 @@ class BatchedDecodeStep:
 
 class StagedItems:
     """One scheduler step as the row arrays its kernels read (device addresses) plus the host-side segment list."""
-    __slots__ = ("n_rows", "n_dec", "n_out", "dec_ctx", "segs", "tokens", "row_slot", "row_pos", "row_off", "out_rows")
+    __slots__ = ("n_rows", "n_dec", "n_out", "n_short", "dec_ctx", "segs", "tokens", "row_slot", "row_pos", "row_off", "out_rows")
 
 
 class ItemStage:
     """Turns ``(slot, start, tokens[, out])`` items into row arrays on the device: single-token items first, then the prompt chunks, each
     row with its slot, position and offset inside its item.  ``out``: how many of the item's last rows are sampled (default 1), or the
-    list of its rows (offsets, ascending) that are.  One pinned staging row and ONE asynchronous copy per step; two of them in turn, each guarded by an
+    list of its rows (offsets, ascending) that are.  ``short``: chunks of up to that many rows come first among the chunks (``n_short`` of them;
+    ``dec_ctx`` covers them too).  One pinned staging row and ONE asynchronous copy per step; two of them in turn, each guarded by an
     event, so that a caller who enqueues steps without synchronising never rewrites a row in flight."""
 
-    def __init__(self, device, n_slots: int, max_len: int, vocab: int):
-        self.dev, self.n_slots, self.max_len, self.vocab = device, int(n_slots), int(max_len), int(vocab)
+    def __init__(self, device, n_slots: int, max_len: int, vocab: int, short: int = 0):
+        self.dev, self.n_slots, self.max_len, self.vocab, self.short = device, int(n_slots), int(max_len), int(vocab), int(short)
         self.rows, self._turn = 0, 0
 
     def ensure(self, rows: int):
@@ -589,7 +590,8 @@ class ItemStage:
             self._ev[sb].synchronize()
         st = self._np[sb]
         tok, rs, rp, ro, outr = st[:R], st[R:2 * R], st[2 * R:3 * R], st[3 * R:4 * R], st[4 * R:]
-        order = sorted(range(n_items), key=lambda i: len(items[i][2]) != 1)          # single-token rows first (stable)
+        kind = lambda n: 0 if n == 1 else 1 if n <= self.short else 2
+        order = sorted(range(n_items), key=lambda i: kind(len(items[i][2])))         # single-token rows first, then short chunks (stable)
         outs = [it[3] if len(it) > 3 else 1 for it in items]
         outs = [list(o) if isinstance(o, (list, tuple)) else list(range(len(it[2]) - int(o), len(it[2]))) for o, it in zip(outs, items)]
         out0, n_out = [], 0
@@ -597,7 +599,7 @@ class ItemStage:
             out0.append(n_out)
             n_out += len(o)
         s = StagedItems()
-        s.segs, row, s.n_dec, s.dec_ctx, seen = [], 0, 0, 0, set()
+        s.segs, row, s.n_dec, s.n_short, s.dec_ctx, seen = [], 0, 0, 0, 0, set()
         for i in order:
             slot, start, toks = items[i][:3]
             n = len(toks)
@@ -614,9 +616,11 @@ class ItemStage:
             ro[row:row + n] = range(n)
             if n == 1:
                 s.n_dec += 1
-                s.dec_ctx = max(s.dec_ctx, start + 1)
             else:
                 s.segs.append((row, n, slot, start))
+                s.n_short += n <= self.short
+            if n == 1 or n <= self.short:
+                s.dec_ctx = max(s.dec_ctx, start + n)
             outr[out0[i]:out0[i] + len(outs[i])] = [row + o for o in outs[i]]
             row += n
         self._d[sb].copy_(self._h[sb], non_blocking=True)                            # stream-ordered before the kernels

@@ -44,7 +44,14 @@ def _load_lebepel(path, device, dtype):
     return load(path, device, dtype)
 
 
+def _load_serotar(path, device, dtype):
+    from .serotar import load
+    return load(path, device, dtype)
+
+
 FAMILIES: List[Family] = [
+    Family("serotar", lambda c: c.get("architecture") == "Serotar", _load_serotar, torch.bfloat16, True, build.LIB_HYBRID,
+           lambda model, n, max_len: model.step_engine(n, max_len), lambda model: model.max_positions),
     Family("lebepel", lambda c: c.get("architecture") == "Lebepel", _load_lebepel, torch.bfloat16, True, build.LIB_HYBRID,
            lambda model, n, max_len: model.step_engine(n, max_len), lambda model: model.max_positions),
     Family("bitllama", lambda c: "architecture" not in c and c.get("model_type", "bitllama") == "bitllama", _load_onebit, torch.float16, False, build.LIB,

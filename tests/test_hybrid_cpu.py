@@ -217,7 +217,7 @@ def test_native_step_rejects_bad_arguments():
         assert size(bad) == 0, (kw, layer)
     seg = (_HSeg * 1)(_HSeg(1, 4, 0, 0))
     def step(mm=m, rows=5, outs=8, **kw):
-        st = _HState(ctypes.sizeof(_HState), 5, 1, 1, 1, 128, 1, a, a, a, a, seg, a, a, a, None, a, 1 << 40)
+        st = _HState(ctypes.sizeof(_HState), 5, 1, 1, 1, 0, 128, 1, a, a, a, a, seg, a, a, a, None, a, 1 << 40)
         for k, v in kw.items():
             setattr(st, k, v)
         return lib.onebit_hybrid_step(ctypes.byref(mm), ctypes.byref(st), rows, outs, 3, 4, None)
