@@ -80,11 +80,38 @@ def hybrid_config(width, layers=8, vocab=32000, max_positions=4096):
                          max_positions=max_positions)
 
 
-def measure_hybrid(dev, what="all", widths=(2048, 4096), beside=True, layers=8):
-    """Prefill and decode throughput of the hybrid decoder at a few sizes, and of the 1-bit LLaMA with the same width, feed-forward, heads and
-    number of layers: prompts through the step engines (``HybridStep`` / ``MixedStep``), decoding by their graphs."""
+# --hybrid-family serotar: width -> (heads, head size, query rank, latent rank, token input); the feed-forward of HYBRID_SIZES as a shared expert
+# (a quarter) and 6 of 32 routed ones (an eighth each) next to 8 identity experts, 4 of 8 groups
+SEROTAR_SIZES = {1024: (16, 64, 384, 128, 32), 2048: (16, 128, 768, 256, 64), 4096: (32, 128, 1536, 512, 128)}
+
+
+def serotar_config(width, layers=8, vocab=32000):
+    from onebit_amd.serotar import SerotarConfig
+    ff = HYBRID_SIZES[width][0]
+    h, d, qr, kr, side = SEROTAR_SIZES[width]
+    mix = {"heads": h, "dim": d, "vdim": d, "q_rank": qr, "kv_rank": kr, "scale": d ** -0.5}
+    moe = {"kind": "moe", "expert": {"ff": ff // 8}, "shared": {"ff": ff // 4}, "router": {"experts": 32, "identity": 8, "top": 6, "groups": {"count": 8, "keep": 4}}}
+    return SerotarConfig(vocab_size=vocab, width=width, norm_eps=1e-5, embed_scale=1.0, bigram={"buckets": 4 * vocab - 1, "mul_prev": 31, "mul_cur": 7}, side_dim=side,
+                         layers=[{"type": "latent_attention", "mixer": mix, "mlp": moe if i else {"kind": "dense", "ff": ff}} for i in range(layers)])
+
+
+def linear_params(cfg):
+    """Weights a row of a hybrid decoder passes through, all layers (of routed experts: the ones it uses, identity experts not counted out)."""
+    total = 0
+    for k, s in cfg.tensor_shapes().items():
+        if k[0] == "l" and k[1].isdigit() and len(s) == 2 and "conv" not in k:
+            lay = cfg.layers[int(k[1:k.index(".")])]
+            r = (lay.get("mlp") or {}).get("router")
+            total += s[0] * s[1] * (r["top"] / r["experts"] if ".mlp.e" in k else 1)
+    return total
+
+
+def measure_hybrid(dev, what="all", widths=(2048, 4096), beside=True, layers=8, family="lebepel"):
+    """Prefill and decode throughput of a hybrid decoder at a few sizes, and beside it of the closest other family with the same width, feed-forward
+    and number of layers (Lebepel: the 1-bit LLaMA; Serotar: Lebepel): prompts through the step engines (``HybridStep`` / ``MixedStep``),
+    decoding by their graphs."""
     from onebit_amd.engine import MixedStep
-    from onebit_amd.lebepel import build_synthetic_model
+    from onebit_amd import lebepel, serotar
     from onebit_amd.llama import OneBitLlamaConfig, KVCache
     from onebit_amd.llama import build_synthetic_model as build_onebit
     from onebit_amd.serving import ContinuousBatcher, Item, Request
@@ -108,13 +135,13 @@ def measure_hybrid(dev, what="all", widths=(2048, 4096), beside=True, layers=8):
     for width in widths:
         ff, ah, ad = HYBRID_SIZES[width][:3]
         row = {"width": width, "ff": ff, "layers": layers}
-        for name in ("lebepel", "onebit_llama") if beside else ("lebepel",):
-            if name == "lebepel":
-                cfg = hybrid_config(width, layers)
-                model = build_synthetic_model(cfg, 1, torch.bfloat16, dev)
-                per_layer = [sum(a * b for a, b in (s for k, s in cfg.tensor_shapes().items() if k.startswith("l%d." % i) and len(s) == 2 and "conv" not in k))
-                             for i in range(2)]
-                flops_row = layers // 2 * sum(per_layer) * 2
+        names = {"lebepel": ("lebepel", "onebit_llama"), "serotar": ("serotar", "lebepel")}[family]
+        for name in names if beside else names[:1]:
+            hybrid = name != "onebit_llama"
+            if hybrid:
+                cfg = hybrid_config(width, layers) if name == "lebepel" else serotar_config(width, layers)
+                model = (lebepel if name == "lebepel" else serotar).build_synthetic_model(cfg, 1, torch.bfloat16, dev)
+                flops_row = 2 * linear_params(cfg)
             else:
                 cfg = OneBitLlamaConfig(vocab_size=32000, hidden_size=width, intermediate_size=ff, num_hidden_layers=layers, num_attention_heads=ah,
                                         max_position_embeddings=4096)
@@ -124,7 +151,7 @@ def measure_hybrid(dev, what="all", widths=(2048, 4096), beside=True, layers=8):
             if what in ("all", "prefill"):
                 for B, S in prompts:
                     toks = [torch.randint(0, 32000, (S,), generator=g).tolist() for _ in range(B)]
-                    if name == "lebepel":
+                    if hybrid:
                         eng = model.step_engine(B, S, max_rows=B * S)
                     else:
                         eng = MixedStep(model, KVCache(cfg, B, S, dev, torch.float16).layers, B, S, max_rows=B * S)
@@ -136,7 +163,7 @@ def measure_hybrid(dev, what="all", widths=(2048, 4096), beside=True, layers=8):
                 for B, ctx in decodes:
                     # steps at a fixed context, enqueued back to back: the engine's graph replay, state and cache holding whatever they hold
                     n_it = 40
-                    if name == "lebepel":
+                    if hybrid:
                         eng = model.step_engine(B, ctx + 8)
                         t = clock(lambda: eng.launch([(b, ctx, [b + 1]) for b in range(B)]), n_it)
                     elif B == 1:
@@ -184,7 +211,8 @@ def parse(argv=None):
                     help="measure the hybrid decoders (Lebepel) beside the 1-bit LLaMA of equal size INSTEAD of the default workload: prefill and "
                          "decode throughput at a few sizes, one JSON line of its own")
     ap.add_argument("--hybrid-size", default="2048,4096", help="widths for --hybrid, comma-separated (of %s)" % ", ".join(map(str, HYBRID_SIZES)))
-    ap.add_argument("--hybrid-only", action="store_true", help="--hybrid without the 1-bit LLaMA beside it (profiles)")
+    ap.add_argument("--hybrid-only", action="store_true", help="--hybrid without the other family beside it (profiles)")
+    ap.add_argument("--hybrid-family", default="lebepel", choices=["lebepel", "serotar"], help="the hybrid decoder to measure: lebepel beside the 1-bit LLaMA, serotar beside lebepel")
     ap.add_argument("--pg-timeout", type=float, default=300.0, help="process-group timeout in seconds (N > 1)")
     return ap.parse_args(argv)
 
@@ -1106,8 +1134,8 @@ def main(argv=None, hooks=None):
     hk = hooks or Hooks()
     if args.hybrid:
         dev = torch.device("cuda:0")
-        rows = measure_hybrid(dev, args.hybrid, [int(w) for w in args.hybrid_size.split(",")], beside=not args.hybrid_only)
-        print(json.dumps({"metric": "hybrid_decoder_throughput", "unit": "tokens/s", "dtype": "bf16 (lebepel) / fp16 + 1-bit weights (onebit_llama)",
+        rows = measure_hybrid(dev, args.hybrid, [int(w) for w in args.hybrid_size.split(",")], beside=not args.hybrid_only, family=args.hybrid_family)
+        print(json.dumps({"metric": "hybrid_decoder_throughput", "unit": "tokens/s", "dtype": "bf16 (lebepel, serotar) / fp16 + 1-bit weights (onebit_llama)",
                           "data": "synthetic", "sizes": rows}))
         return
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:

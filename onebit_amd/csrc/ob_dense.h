@@ -76,7 +76,7 @@ template <typename E> __device__ __forceinline__ float ob_gelu_tanh(float z)
 {
     const float u = 0.79788456080286536f * (z + 0.044715f * z * z * z);
     if constexpr (sizeof(E) == 2) return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-2.8853900817779268f * u));
-    else return 0.5f * z * (1.0f + tanhf(u));
+    else return z * ob_sigmoidf(2.0f * u);
 }
 // quadratic above zero, exponential below, slope 1/2 at zero:  a z^2 + z / 2  |  b (e^z - 1 - z) + z / 2
 template <typename E> __device__ __forceinline__ float ob_xielu(float z, float a, float b)

@@ -149,7 +149,7 @@ def synthetic_weights(cfg: SerotarConfig, seed: int = 0, dtype=torch.bfloat16, d
     """Random weights of the configuration's shapes: linears N(0, 1 / fan_in), norms and layer scales around one, depth weights around keeping the
     last result."""
     g = torch.Generator(device=device).manual_seed(seed)
-    rnd = lambda *s: torch.randn(*s, generator=g, device=device)
+    rnd = lambda *s: torch.randn(s, generator=g, device=device)
     out = {}
     for name, shape in cfg.tensor_shapes().items():
         leaf = name.rsplit(".", 1)[-1]
