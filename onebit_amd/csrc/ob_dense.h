@@ -94,19 +94,20 @@ __device__ __forceinline__ float ob_softplusf(float z) { return fmaxf(z, 0.0f) +
 //                 fragment-major rows of the output product, at column act_k0
 //   OB_EPI_PART   fp32 partial sums z[split][t][n] (the layer's output product: the row kernel that follows adds the splits)
 //   OB_EPI_LOGITS fp32 logits[t][n], cap * tanh(v / cap) when cap > 0
-//   OB_EPI_ACT    f(v) into fragment-major rows at column act_k0 + n: f = identity, xIELU, or gelu_tanh(v) times an entry of the token's row
-//                 of a table
+//   OB_EPI_ACT    f(v) into fragment-major rows at column act_k0 + n: f = identity or xIELU
 //   OB_EPI_HEADS  head-major rows: heads[n / D][t][n % D] (D a power of two), keys and values of a prompt's latents
-enum ObEpilogue { OB_EPI_IN = 0, OB_EPI_PART = 1, OB_EPI_LOGITS = 2, OB_EPI_ACT = 3, OB_EPI_HEADS = 4 };
-enum ObDenseFn { OB_FN_ID = 0, OB_FN_XIELU = 1, OB_FN_GELU_TABLE = 2 };
+//   OB_EPI_QFRAG  per token and 16 heads (columns n = head D + r) the operand tiles of a score product, heads as its rows: bf16
+enum ObEpilogue { OB_EPI_IN = 0, OB_EPI_PART = 1, OB_EPI_LOGITS = 2, OB_EPI_ACT = 3, OB_EPI_HEADS = 4, OB_EPI_QFRAG = 5 };
+enum ObDenseFn { OB_FN_ID = 0, OB_FN_XIELU = 1 };
 
 // ---- which weights meet which rows ------------------------------------------------------------------------------------------
 //   OB_ROWS_ALL     every row, fragment-major activations
 //   OB_ROWS_HEADS   block-diagonal over heads: n tiles tile_group apart read their own act_cols columns of ROW-MAJOR activations
 //   OB_ROWS_GATHER  blocks of one expert's rows (ObRowBlock table): activation row gather[row] of a ROW-MAJOR matrix, output row `row`
 //   OB_ROWS_SORTED  the same blocks, fragment-major activations in block order
+//   OB_ROWS_TABLE   few rows, formed here: gelu_tanh(sum of `n_pre` partial sums of another product) times the token's row of a table
 //   OB_ROWS_SEGS    rows of several requests' cache slots (fragment-major bands), output rows consecutive per request
-enum ObRowForm { OB_ROWS_ALL = 0, OB_ROWS_HEADS = 1, OB_ROWS_GATHER = 2, OB_ROWS_SORTED = 3, OB_ROWS_SEGS = 4 };
+enum ObRowForm { OB_ROWS_ALL = 0, OB_ROWS_HEADS = 1, OB_ROWS_GATHER = 2, OB_ROWS_SORTED = 3, OB_ROWS_SEGS = 4, OB_ROWS_TABLE = 5 };
 struct ObRowBlock { int32_t group, row0, count, pad; };      // rows [row0, row0 + count) of weight group `group`; row0 a multiple of 16 at a group's start
 
 struct ObDenseArgs {
@@ -124,11 +125,13 @@ struct ObDenseArgs {
     float *logits; int V; float cap;
     // OB_EPI_ACT (act, act_k0, act_nkt as above)
     int fn; float fa, fb;          // xIELU's two factors
-    const void *table; const int32_t *tokens; int ld_table, table_cols;      // entry (tokens[t], n), n < table_cols
-    // OB_EPI_HEADS
+    // OB_EPI_HEADS, OB_EPI_QFRAG (D = 1 << d_shift; head_rows: rows per head / tiles of 16 heads)
     void *heads; int d_shift, head_rows;
     // OB_ROWS_HEADS / OB_ROWS_GATHER: row-major activations
     int lda, tile_group, act_cols;
+    // OB_ROWS_TABLE: pre [n_pre][T][ld_pre] fp32, columns nkt KT
+    const float *pre; int n_pre, ld_pre;
+    const void *table; const int32_t *tokens; int ld_table, table_cols;      // entry (tokens[t], n), n < table_cols
     // OB_ROWS_GATHER / OB_ROWS_SORTED
     const ObRowBlock *blk; const int32_t *gather; size_t w_group;             // weight tiles per group
 };
@@ -148,23 +151,22 @@ template <typename E, int EPI>
 __device__ __forceinline__ void ob_dense_epilogue(const ObDenseArgs &A, int nt, int t, bool live, int g, ob_float4 v0, ob_float4 v1, int split)
 {
     if (!live) return;
-    if constexpr (EPI == OB_EPI_ACT || EPI == OB_EPI_HEADS) {
+    if constexpr (EPI == OB_EPI_ACT || EPI == OB_EPI_HEADS || EPI == OB_EPI_QFRAG) {
 #pragma unroll
         for (int h = 0; h < 2; ++h) {
             if (nt + h >= A.n_tiles) return;
             ob_float4 v = h ? v1 : v0;
             const int n = (nt + h) * 16 + 4 * g;
-            if constexpr (EPI == OB_EPI_HEADS) {
+            if constexpr (EPI == OB_EPI_QFRAG) {
+                const int hd = n >> A.d_shift, r = n & ((1 << A.d_shift) - 1);
+                *reinterpret_cast<typename ObElem<E>::V4 *>((E *)A.heads + ((((size_t)t * A.head_rows + (hd >> 4)) << (A.d_shift + 4)) + ob_frag<E>(hd & 15, r, 0))) = ob_to_v4<E>(v);
+            } else if constexpr (EPI == OB_EPI_HEADS) {
                 const int hd = n >> A.d_shift, d = n & ((1 << A.d_shift) - 1);
                 *reinterpret_cast<typename ObElem<E>::V4 *>((E *)A.heads + ((((size_t)hd * A.head_rows + t) << A.d_shift) + d)) = ob_to_v4<E>(v);
             } else {
                 if (A.fn == OB_FN_XIELU) {
 #pragma unroll
                     for (int e = 0; e < 4; ++e) v[e] = ob_xielu<E>(v[e], A.fa, A.fb);
-                } else if (A.fn == OB_FN_GELU_TABLE) {
-                    const E *row = (const E *)A.table + (size_t)A.tokens[t] * A.ld_table;
-#pragma unroll
-                    for (int e = 0; e < 4; ++e) v[e] = n + e < A.table_cols ? ob_gelu_tanh<E>(v[e]) * (float)row[n + e] : 0.f;
                 }
                 *reinterpret_cast<typename ObElem<E>::V4 *>((E *)A.act + ob_frag<E>(t, A.act_k0 + n, A.act_nkt)) = ob_to_v4<E>(v);
             }
@@ -214,6 +216,33 @@ __device__ __forceinline__ void ob_dense_epilogue(const ObDenseArgs &A, int nt, 
     }
 }
 
+// four columns of a row of the OB_ROWS_TABLE operand
+template <typename E> __device__ __forceinline__ void ob_table_piece(const ObDenseArgs &A, E *dst, int t, int n)
+{
+    const float *zp = A.pre + (size_t)t * A.ld_pre + n;
+    const E *row = (const E *)A.table + (size_t)A.tokens[t] * A.ld_table + n;
+    ob_float4 v = {0.f, 0.f, 0.f, 0.f}, tv = v;
+    for (int k = 0; k < A.n_pre; k += 4) {                             // four splits in flight, added in order
+        ob_float4 zv[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) zv[j] = *reinterpret_cast<const ob_float4 *>(zp + (size_t)min(k + j, A.n_pre - 1) * A.T * A.ld_pre);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) if (k + j < A.n_pre) v += zv[j];
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) if (n + e < A.table_cols) tv[e] = (float)row[e];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = n + e < A.table_cols ? ob_gelu_tanh<E>(v[e]) * tv[e] : 0.f;
+    *reinterpret_cast<typename ObElem<E>::V4 *>(dst + ob_frag<E>(t, n, A.nkt)) = ob_to_v4<E>(v);
+}
+// ... of many rows, in memory: grid (pieces / 256)
+template <typename E> __global__ __launch_bounds__(256) void ob_table_rows_kernel(const ObDenseArgs A)
+{
+    const int nv = A.nkt * ObElem<E>::KT / 4;
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i < (int64_t)A.T * nv) ob_table_piece<E>(A, (E *)A.act, (int)(i / nv), 4 * (int)(i % nv));
+}
+
 // ---- few rows (T <= 64): weights from HBM straight into the operand registers ------------------------------------------
 // Workgroup = 2 n tiles (32 output columns; a gate / up pair) x all token tiles x one K split; its four waves take a quarter of the
 // split's k tiles each and add up through LDS.  Activations come from L2 (1 KB linear loads).  The next U k tiles are requested
@@ -226,6 +255,7 @@ __global__ __launch_bounds__(256, MT >= 4 ? 2 : 3) void ob_dense_skinny_kernel(c
     typedef typename ObElem<E>::V16 V16;
     constexpr int U = MT >= 4 ? 2 : 4;
     __shared__ ob_float4 red[4][2][MT][64];
+    extern __shared__ __attribute__((aligned(16))) char formed[];      // OB_ROWS_TABLE: [MT][nkt] tiles
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int nt = blockIdx.x * 2, split = blockIdx.y;
     const int k_lo = split * A.kt_split, k_hi = min(A.nkt, k_lo + A.kt_split);
@@ -240,6 +270,11 @@ __global__ __launch_bounds__(256, MT >= 4 ? 2 : 3) void ob_dense_skinny_kernel(c
     }
     const V16 *w0 = (const V16 *)A.w + (wg + (size_t)nt * A.nkt) * 64 + lane;
     const V16 *w1 = (const V16 *)A.w + (wg + (size_t)min(nt + 1, A.n_tiles - 1) * A.nkt) * 64 + lane;
+    if constexpr (ROWS == OB_ROWS_TABLE) {
+        const int nv = A.nkt * ObElem<E>::KT / 4;
+        for (int i = tid; i < A.T * nv; i += 256) ob_table_piece<E>(A, (E *)formed, i / nv, 4 * (i % nv));
+        __syncthreads();
+    }
     // this lane's piece of k tile 0 of every token tile, and the step (in 16 bytes) to the next k tile
     const V16 *ap[MT];
     constexpr int KSTEP = ROWS == OB_ROWS_HEADS || ROWS == OB_ROWS_GATHER ? 4 : 64;
@@ -249,6 +284,7 @@ __global__ __launch_bounds__(256, MT >= 4 ? 2 : 3) void ob_dense_skinny_kernel(c
             ap[m] = (const V16 *)((const E *)A.a + (size_t)min(m * 16 + (lane & 15), rows - 1) * A.lda + nt / A.tile_group * A.act_cols) + (lane >> 4);
         else if constexpr (ROWS == OB_ROWS_GATHER)
             ap[m] = (const V16 *)((const E *)A.a + (size_t)A.gather[t0 + min(m * 16 + (lane & 15), rows - 1)] * A.lda) + (lane >> 4);
+        else if constexpr (ROWS == OB_ROWS_TABLE) ap[m] = (const V16 *)formed + lane + (size_t)m * A.nkt * 64;
         else ap[m] = (const V16 *)A.a + lane + (size_t)((t0 >> 4) + m) * A.nkt * 64;
     }
     ob_float4 acc[2][MT];

@@ -3,6 +3,25 @@
 #pragma once
 #include "ob_dense.h"
 
+// s += sum of n partial sums `stride` apart: four in flight, added in order
+template <int VEC>
+__device__ __forceinline__ void ob_sum_splits(float (&s)[VEC], const float *p, size_t stride, int n)
+{
+    for (int k = 0; k < n; k += 4) {
+        float zv[4][VEC];
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) zv[j][e] = p[(size_t)min(k + j, n - 1) * stride + e];
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+            if (k + j < n) {
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) s[e] += zv[j][e];
+            }
+    }
+}
+
 // r = residual row, formed one of two ways; x (fragment-major, the next product's operand) = r / sqrt(mean r^2 + eps) * (off + w)
 //   embed != NULL   r = embed[token] (+ pos_embed[position]); copied to emb_save when given
 //   else            r = x_in + mult * (sum of the splits of the output product + bias) (+ emb_add: a looped stretch starting over)
@@ -41,20 +60,7 @@ __global__ __launch_bounds__(1024) void ob_hnorm_kernel(const ObHNormArgs A)
             float s[VEC], xv[VEC];
 #pragma unroll
             for (int e = 0; e < VEC; ++e) { s[e] = 0.f; xv[e] = xr[c + e]; }
-            const float *zr = A.z + (size_t)src * A.ldz + c;
-            for (int k = 0; k < A.n_split; k += 4) {                  // four splits in flight, added in order
-                float zv[4][VEC];
-#pragma unroll
-                for (int j = 0; j < 4; ++j)
-#pragma unroll
-                    for (int e = 0; e < VEC; ++e) zv[j][e] = zr[(size_t)min(k + j, A.n_split - 1) * A.z_split + e];
-#pragma unroll
-                for (int j = 0; j < 4; ++j)
-                    if (k + j < A.n_split) {
-#pragma unroll
-                        for (int e = 0; e < VEC; ++e) s[e] += zv[j][e];
-                    }
-            }
+            ob_sum_splits<VEC>(s, A.z + (size_t)src * A.ldz + c, A.z_split, A.n_split);
 #pragma unroll
             for (int e = 0; e < VEC; ++e) r[e] = xv[e] + A.mult * (A.bias ? s[e] + A.bias[c + e] : s[e]);
             if (A.emb_add) {
@@ -87,7 +93,7 @@ __global__ __launch_bounds__(1024) void ob_hnorm_kernel(const ObHNormArgs A)
 }
 
 // The same row with everything a sequential layer adds to it:
-//   s = sum of the splits (+ bias) + sum_k tok_w[k] ez[tok_row[k]] (experts) + id_w h (identity experts; h = idh or the residual itself)
+//   s = sum of the splits (+ bias) + sum_k tok_w[k] ez[tok_row[k]] (experts; eo: their outputs in the work type) + id_w h (identity experts; h = idh or the residual itself)
 //   r = x + mult * (post_w ? s / sqrt(mean s^2 + eps) * post_w : s) (+ emb_add)
 //     or, embed != NULL: r = embed[token] * embed_scale (+ bigram[row of (previous token, token)]) (+ pos_embed[position])
 //   hist: X_i = r is kept (i = hist_i), and with dwa the stream goes on as sum_j dwa[j] X_j, j = 0 .. hist_i
@@ -97,37 +103,26 @@ struct ObXRowArgs : ObHNormArgs {
     float embed_scale; const void *bigram; int buckets, mul_prev, mul_cur;
     int32_t *tok_hist; const int32_t *row_slot, *row_off; int n_slots, max_len;
     const float *post_w;
-    const float *ez; size_t ez_split; int ez_n, ld_ez, top; const int32_t *tok_row; const float *tok_w, *id_w; const void *idh; int ld_idh;
+    const float *ez; const void *eo; size_t ez_split; int ez_n, ld_ez, top; const int32_t *tok_row; const float *tok_w, *id_w; const void *idh; int ld_idh;
     float *hist; size_t hist_stride; int hist_i; const float *dwa;
     void *out_rm; int ld_rm;
 };
-template <typename E, int VEC>
-__device__ __forceinline__ void ob_sum_splits(float (&s)[VEC], const float *p, size_t stride, int n)
-{
-    for (int k = 0; k < n; k += 4) {                                  // four splits in flight, added in order
-        float zv[4][VEC];
-#pragma unroll
-        for (int j = 0; j < 4; ++j)
-#pragma unroll
-            for (int e = 0; e < VEC; ++e) zv[j][e] = p[(size_t)min(k + j, n - 1) * stride + e];
-#pragma unroll
-        for (int j = 0; j < 4; ++j)
-            if (k + j < n) {
-#pragma unroll
-                for (int e = 0; e < VEC; ++e) s[e] += zv[j][e];
-            }
-    }
-}
-template <typename E, int VEC>
+// ONE: a thread has one piece of the row (W <= threads * VEC); everything that does not depend on the first reduction is then requested before it.
+// KIND: what can be there besides the sum of splits (smaller code: at a few rows a launch's time is its chain of fetches, instructions included)
+enum ObXKind { OB_X_PLAIN = 0, OB_X_EXPERTS = 1, OB_X_DEPTH = 2, OB_X_BOTH = 3, OB_X_EMBED = 4 };
+template <typename E, int VEC, bool ONE, int KIND>
 __global__ __launch_bounds__(1024) void ob_xrow_kernel(const ObXRowArgs A)
 {
+    constexpr int NH = 8;
+    constexpr bool EMB = KIND == OB_X_EMBED, EXP = (KIND & 1) != 0, DEP = (KIND & 2) != 0;
     extern __shared__ __attribute__((aligned(16))) float sm[];        // [W] row | [16] reduction
     float *red = sm + ((A.W + 3) & ~3);
     const int t = blockIdx.x, tid = threadIdx.x, stride = blockDim.x * VEC;
     const int src = A.rows ? A.rows[t] : t;
     float *xr = A.x + (size_t)src * A.W;
+    float *hr = A.hist + (size_t)src * A.W;                           // (DEP, and EMB where the embedding is kept)
     const E *er = nullptr, *pr = nullptr, *br = nullptr;
-    if (A.embed) {
+    if constexpr (EMB) {
         const int tok = A.tokens[src], pos = A.row_pos[src], slot = A.row_slot[src];
         er = (const E *)A.embed + (size_t)tok * A.W;
         if (A.pos_embed) pr = (const E *)A.pos_embed + (size_t)max(pos, 0) * A.W;
@@ -142,73 +137,109 @@ __global__ __launch_bounds__(1024) void ob_xrow_kernel(const ObXRowArgs A)
             if (live && tid == 0 && !A.rows) A.tok_hist[(size_t)slot * A.max_len + pos] = tok;
         }
     }
+    float x1[VEC], h1[DEP ? NH : 1][VEC];                             // ONE: the residual and the first results X_j
+    if (ONE && !EMB && tid * VEC < A.W) {
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) x1[e] = xr[tid * VEC + e];
+        if (DEP && A.dwa) {
+#pragma unroll
+            for (int j = 0; j < NH; ++j)
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) h1[DEP ? j : 0][e] = hr[(size_t)min(j, A.hist_i - 1) * A.hist_stride + tid * VEC + e];
+        }
+    }
     float ss = 0.f;
-    if (!er) {
+    if (!EMB) {
         for (int c = tid * VEC; c < A.W; c += stride) {
             float s[VEC];
 #pragma unroll
             for (int e = 0; e < VEC; ++e) s[e] = 0.f;
-            if (A.z) ob_sum_splits<E, VEC>(s, A.z + (size_t)src * A.ldz + c, A.z_split, A.n_split);
+            if (A.z) ob_sum_splits<VEC>(s, A.z + (size_t)src * A.ldz + c, A.z_split, A.n_split);
             if (A.bias) {
 #pragma unroll
                 for (int e = 0; e < VEC; ++e) s[e] += A.bias[c + e];
             }
-            if (A.ez) {
-                for (int k = 0; k < A.top; ++k) {
-                    const int row = A.tok_row[(size_t)src * A.top + k];                    // (uniform)
-                    if (row < 0) continue;
-                    const float w = A.tok_w[(size_t)src * A.top + k];
-                    float y[VEC];
+            if (EXP && A.eo) {                                        // four experts in flight, added in order
+#pragma unroll 1
+                for (int k0 = 0; k0 < A.top; k0 += 4) {
+                    float y[4][VEC], w[4];
 #pragma unroll
-                    for (int e = 0; e < VEC; ++e) y[e] = 0.f;
-                    ob_sum_splits<E, VEC>(y, A.ez + (size_t)row * A.ld_ez + c, A.ez_split, A.ez_n);
+                    for (int j = 0; j < 4; ++j) {
+                        const size_t k = (size_t)src * A.top + min(k0 + j, A.top - 1);
+                        const int row = A.tok_row[k];                 // (uniform; row 0 where there is none)
+                        w[j] = k0 + j < A.top && row >= 0 ? A.tok_w[k] : 0.f;
+                        const E *p = (const E *)A.eo + (size_t)max(row, 0) * A.ld_ez + c;
 #pragma unroll
-                    for (int e = 0; e < VEC; ++e) s[e] = __builtin_fmaf(w, y[e], s[e]);
+                        for (int e = 0; e < VEC; ++e) y[j][e] = (float)p[e];
+                    }
+#pragma unroll
+                    for (int j = 0; j < 4; ++j)
+#pragma unroll
+                        for (int e = 0; e < VEC; ++e) s[e] = w[j] != 0.f ? __builtin_fmaf(w[j], y[j][e], s[e]) : s[e];
+                }
+            } else if (EXP) {
+#pragma unroll 1
+                for (int k0 = 0; k0 < A.top * A.ez_n; k0 += 4) {      // (choice, split) pairs
+                    float y[4][VEC], w[4];
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) {
+                        const int kk = min(k0 + j, A.top * A.ez_n - 1), sp = A.ez_n == 1 ? 0 : kk / A.top;
+                        const size_t k = (size_t)src * A.top + kk - sp * A.top;
+                        const int row = A.tok_row[k];
+                        w[j] = k0 + j < A.top * A.ez_n && row >= 0 ? A.tok_w[k] : 0.f;
+                        const float *p = A.ez + sp * A.ez_split + (size_t)max(row, 0) * A.ld_ez + c;
+#pragma unroll
+                        for (int e = 0; e < VEC; ++e) y[j][e] = p[e];
+                    }
+#pragma unroll
+                    for (int j = 0; j < 4; ++j)
+#pragma unroll
+                        for (int e = 0; e < VEC; ++e) s[e] = w[j] != 0.f ? __builtin_fmaf(w[j], y[j][e], s[e]) : s[e];
                 }
             }
-            if (A.id_w) {
+            if (EXP && A.id_w) {
                 const float w = A.id_w[src];
 #pragma unroll
-                for (int e = 0; e < VEC; ++e) s[e] = __builtin_fmaf(w, A.idh ? (float)((const E *)A.idh)[(size_t)src * A.ld_idh + c + e] : xr[c + e], s[e]);
+                for (int e = 0; e < VEC; ++e)
+                    s[e] = __builtin_fmaf(w, A.idh ? (float)((const E *)A.idh)[(size_t)src * A.ld_idh + c + e] : ONE ? x1[e] : xr[c + e], s[e]);
             }
 #pragma unroll
             for (int e = 0; e < VEC; ++e) { sm[c + e] = s[e]; ss = __builtin_fmaf(s[e], s[e], ss); }
         }
     }
     float rp = 1.f;
-    if (A.post_w) rp = 1.0f / sqrtf(ob_block_sum(ss, red) / (float)A.W + A.eps);          // (uniform)
+    if (!EMB && A.post_w) rp = 1.0f / sqrtf(ob_block_sum(ss, red) / (float)A.W + A.eps);          // (uniform)
     ss = 0.f;
     for (int c = tid * VEC; c < A.W; c += stride) {
         float r[VEC];
-        if (er) {
+        if (EMB) {
 #pragma unroll
             for (int e = 0; e < VEC; ++e) r[e] = (float)er[c + e] * A.embed_scale + (br ? (float)br[c + e] : 0.f) + (pr ? (float)pr[c + e] : 0.f);
         } else {
 #pragma unroll
-            for (int e = 0; e < VEC; ++e) r[e] = xr[c + e] + A.mult * (A.post_w ? sm[c + e] * rp * A.post_w[c + e] : sm[c + e]);
+            for (int e = 0; e < VEC; ++e) r[e] = (ONE ? x1[e] : xr[c + e]) + A.mult * (A.post_w ? sm[c + e] * rp * A.post_w[c + e] : sm[c + e]);
             if (A.emb_add) {
 #pragma unroll
                 for (int e = 0; e < VEC; ++e) r[e] += A.emb_add[(size_t)src * A.W + c + e];
             }
         }
-        if (A.hist) {
-            float *hr = A.hist + (size_t)src * A.W + c;
+        if (DEP || (EMB && A.hist)) {
             if (!A.rows) {
 #pragma unroll
-                for (int e = 0; e < VEC; ++e) hr[A.hist_i * A.hist_stride + e] = r[e];
+                for (int e = 0; e < VEC; ++e) hr[A.hist_i * A.hist_stride + c + e] = r[e];
             }
-            if (A.dwa) {
+            if (DEP && A.dwa) {
                 float a[VEC];
 #pragma unroll
                 for (int e = 0; e < VEC; ++e) a[e] = 0.f;
-                for (int j = 0; j < A.hist_i; j += 4) {
-                    float v[4][VEC];
+                for (int j = 0; j < A.hist_i; j += NH) {              // eight results in flight, added in order
+                    float v[NH][VEC];
 #pragma unroll
-                    for (int q = 0; q < 4; ++q)
+                    for (int q = 0; q < NH; ++q)
 #pragma unroll
-                        for (int e = 0; e < VEC; ++e) v[q][e] = hr[min(j + q, A.hist_i - 1) * A.hist_stride + e];
+                        for (int e = 0; e < VEC; ++e) v[q][e] = ONE && j == 0 ? h1[DEP ? q : 0][e] : hr[(size_t)min(j + q, A.hist_i - 1) * A.hist_stride + c + e];
 #pragma unroll
-                    for (int q = 0; q < 4; ++q)
+                    for (int q = 0; q < NH; ++q)
                         if (j + q < A.hist_i) {
 #pragma unroll
                             for (int e = 0; e < VEC; ++e) a[e] = __builtin_fmaf(A.dwa[j + q], v[q][e], a[e]);

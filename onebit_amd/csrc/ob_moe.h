@@ -17,55 +17,70 @@ struct ObRouteArgs {
     int32_t *hist;                             // [workgroups][experts]
     int32_t *gather; ObRowBlock *blk; int block_rows, n_blk;
 };
-static inline size_t ob_route_lds(const ObRouteArgs &A) { return ((size_t)16 * (A.experts + A.identity) + 16 * A.groups) * 4 + (size_t)A.experts * 4; }
+// LDS of the first pass: per wave [groups] group maxima; [experts] counts; [64 top] experts of the workgroup's tokens
+static inline size_t ob_route_lds(const ObRouteArgs &A) { return (16 * (size_t)A.groups + A.experts + (size_t)OB_MOE_TOKENS * A.top) * 4; }
+#define OB_MOE_MAX 1024               // experts + identity experts
 
-// one wave per token: choice scores in LDS, every lane ranks its own entries against all others
-__device__ __forceinline__ void ob_route_token(const ObRouteArgs &A, int t, float *cs, float *gs, int lane)
+// order-preserving integers: the largest of a group through an LDS atomic
+__device__ __forceinline__ uint32_t ob_ordered(float v) { const uint32_t u = __float_as_uint(v); return u & 0x80000000u ? ~u : u | 0x80000000u; }
+
+// one wave per token, entry i = lane + 64 j in registers; z: its logits (-inf beyond N)
+template <int NJ>
+__device__ __forceinline__ void ob_route_token(const ObRouteArgs &A, int t, const float (&z)[NJ], const float (&corr)[NJ], uint32_t *gs, int *slots, int lane)
 {
-    const int N = A.experts + A.identity, per = N / A.groups;
-    const float *z = A.z + (size_t)t * A.ldz;
-    float mx = -INFINITY;
-    for (int i = lane; i < N; i += 64) mx = fmaxf(mx, z[i]);
+    const int N = A.experts + A.identity;
+    float mx = z[0];
+#pragma unroll
+    for (int j = 1; j < NJ; ++j) mx = fmaxf(mx, z[j]);
     mx = ob_wave_max(mx);
-    float sum = 0.f;
-    for (int i = lane; i < N; i += 64) sum += expf(z[i] - mx);
-    sum = ob_wave_sum(sum);
-    auto score = [&](int i) { return expf(z[i] - mx) / sum; };
-    for (int i = lane; i < N; i += 64) cs[i] = score(i) + A.correction[i];
-    for (int k = lane; k < A.top; k += 64) { A.tok_row[(size_t)t * A.top + k] = -1; A.tok_w[(size_t)t * A.top + k] = 0.f; }
-    __builtin_amdgcn_wave_barrier();
-    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");       // (this wave's LDS and the cleared slots)
+    float p[NJ], c[NJ], sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) { p[j] = expf(z[j] - mx); sum += p[j]; }
+    const float inv = 1.0f / ob_wave_sum(sum);
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) { p[j] *= inv; c[j] = lane + 64 * j < N ? p[j] + corr[j] : -INFINITY; }
     if (A.keep < A.groups) {
-        for (int g = lane; g < A.groups; g += 64) {
-            float m = -INFINITY;
-            for (int i = 0; i < per; ++i) m = fmaxf(m, cs[g * per + i]);
-            gs[g] = m;
+        const float per_inv = (float)A.groups / (float)N;
+        auto fence = [] { __builtin_amdgcn_wave_barrier(); asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory"); };
+        auto group = [&](int j) { return (int)(((float)(lane + 64 * j) + 0.5f) * per_inv); };         // (lane + 64 j) / (N / groups)
+        for (int g = lane; g < A.groups; g += 64) gs[g] = 0;
+        fence();
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) if (lane + 64 * j < N) atomicMax(&gs[group(j)], ob_ordered(c[j]));
+        fence();
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) {
+            if (lane + 64 * j >= N) continue;
+            const int g = group(j);
+            const uint32_t mine = gs[g];
+            int r = 0;
+            for (int o = 0; o < A.groups; ++o) r += gs[o] > mine || (gs[o] == mine && o < g);
+            if (r >= A.keep) c[j] = -INFINITY;
         }
-        __builtin_amdgcn_wave_barrier();
-        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     }
-    auto allowed = [&](int i) {
-        if (A.keep >= A.groups) return true;
-        const int g = i / per;
-        int r = 0;
-        for (int o = 0; o < A.groups; ++o) r += gs[o] > gs[g] || (gs[o] == gs[g] && o < g);
-        return r < A.keep;
-    };
-    for (int i = lane; i < N; i += 64) if (!allowed(i)) cs[i] = -INFINITY;
-    __builtin_amdgcn_wave_barrier();
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     float idw = 0.f;
-    for (int i = lane; i < N; i += 64) {
-        const float c = cs[i];
-        if (c == -INFINITY) continue;
-        int r = 0;
-        for (int o = 0; o < N; ++o) r += cs[o] > c || (cs[o] == c && o < i);
-        if (r >= A.top) continue;
-        const float w = score(i);
-        if (i >= A.experts) idw += w;
-        else { A.tok_row[(size_t)t * A.top + r] = i; A.tok_w[(size_t)t * A.top + r] = w; }
+    for (int k = 0; k < A.top; ++k) {
+        float best = c[0];
+#pragma unroll
+        for (int j = 1; j < NJ; ++j) best = fmaxf(best, c[j]);
+        best = ob_wave_max(best);
+        int at = -1;                                                  // the smallest index among equals (uniform); none left: -1
+        float w = 0.f;
+        if (best > -INFINITY) {
+#pragma unroll
+            for (int j = 0; j < NJ; ++j) {
+                const uint64_t b = at < 0 ? __builtin_amdgcn_ballot_w64(c[j] == best) : 0;
+                if (b) {
+                    const int l = __builtin_ctzll(b);
+                    at = l + 64 * j;
+                    w = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, p[j]), l));
+                    if (lane == l) c[j] = -INFINITY;
+                }
+            }
+        }
+        if (at >= A.experts) { idw += w; at = -1; }
+        if (lane == 0) { slots[k] = at; A.tok_w[(size_t)t * A.top + k] = w; }
     }
-    idw = ob_wave_sum(idw);
     if (lane == 0) A.id_w[t] = idw;
 }
 
@@ -101,66 +116,91 @@ __device__ __forceinline__ void ob_route_offsets(const ObRouteArgs &A, int *cnt,
 }
 
 // first pass: choices, weights, and this workgroup's tokens per expert.  SINGLE: up to 64 tokens in one workgroup, everything in one launch.
-template <bool SINGLE>
+template <bool SINGLE, int NJ>
 __global__ __launch_bounds__(1024) void ob_route_kernel(const ObRouteArgs A)
 {
-    extern __shared__ __attribute__((aligned(16))) float sm[];        // [16][N] choices | [16][groups] | [experts] counts
+    extern __shared__ __attribute__((aligned(16))) float sm[];
     __shared__ int scan[32];
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, N = A.experts + A.identity;
-    float *cs = sm + (size_t)wave * N, *gs = sm + (size_t)16 * N + wave * A.groups;
-    int *cnt = reinterpret_cast<int *>(sm + (size_t)16 * N + 16 * A.groups);
+    constexpr int PER = NJ <= 4 ? OB_MOE_TOKENS / 16 : 1;             // a wave's tokens whose logits are requested together
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), N = A.experts + A.identity;
+    uint32_t *gs = reinterpret_cast<uint32_t *>(sm) + wave * A.groups;
+    int *cnt = reinterpret_cast<int *>(sm) + 16 * A.groups, *slots = cnt + A.experts;
     for (int e = tid; e < A.experts; e += 1024) cnt[e] = 0;
-    const int t0 = blockIdx.x * OB_MOE_TOKENS, t1 = min(A.T, t0 + OB_MOE_TOKENS);
-    for (int t = t0 + wave; t < t1; t += 16) {
-        ob_route_token(A, t, cs, gs, lane);
-        __builtin_amdgcn_wave_barrier();
+    const int t0 = blockIdx.x * OB_MOE_TOKENS, t1 = min(A.T, t0 + OB_MOE_TOKENS), n = (t1 - t0) * A.top;
+    float corr[NJ];
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) corr[j] = lane + 64 * j < N ? A.correction[lane + 64 * j] : 0.f;
+    for (int tb = t0 + wave; tb < t1; tb += 16 * PER) {
+        float z[PER][NJ];
+#pragma unroll
+        for (int q = 0; q < PER; ++q)
+#pragma unroll
+            for (int j = 0; j < NJ; ++j)
+                z[q][j] = tb + 16 * q < t1 && lane + 64 * j < N ? A.z[(size_t)(tb + 16 * q) * A.ldz + lane + 64 * j] : -INFINITY;
+#pragma unroll 1
+        for (int q = 0; q < PER; ++q) {
+            const int t = tb + 16 * q;
+            if (t >= t1) break;
+            ob_route_token<NJ>(A, t, z[0], corr, gs, slots + (t - t0) * A.top, lane);
+#pragma unroll
+            for (int s = 0; s + 1 < PER; ++s)                         // (the next token's logits move up: one copy of the code)
+#pragma unroll
+                for (int j = 0; j < NJ; ++j) z[s][j] = z[s + 1][j];
+        }
     }
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    __syncthreads();                                                  // (the slots are read back by other lanes of this workgroup: same CU)
-    for (int i = t0 * A.top + tid; i < t1 * A.top; i += 1024) {
-        const int e = __hip_atomic_load(A.tok_row + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_WORKGROUP);
-        if (e >= 0) atomicAdd(&cnt[e], 1);
-    }
+    __syncthreads();
+    for (int i = tid; i < n; i += 1024) if (slots[i] >= 0) atomicAdd(&cnt[slots[i]], 1);
     __syncthreads();
     if constexpr (!SINGLE) {
         for (int e = tid; e < A.experts; e += 1024) A.hist[(size_t)blockIdx.x * A.experts + e] = cnt[e];
+        for (int i = tid; i < n; i += 1024) A.tok_row[(size_t)t0 * A.top + i] = slots[i];
     } else {
         ob_route_offsets(A, cnt, scan, tid);
         __syncthreads();
-        for (int i = tid; i < A.T * A.top; i += 1024) {
-            const int e = __hip_atomic_load(A.tok_row + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_WORKGROUP);
-            if (e < 0) continue;
-            const int r = atomicAdd(&cnt[e], 1);                      // (the order within an expert is free: every row is computed alone)
-            A.gather[r] = i / A.top;
+        for (int i = tid; i < n; i += 1024) {
+            int r = -1;
+            if (slots[i] >= 0) {
+                r = atomicAdd(&cnt[slots[i]], 1);                     // (the order within an expert is free: every row is computed alone)
+                A.gather[r] = i / A.top;
+            }
             A.tok_row[i] = r;
         }
     }
 }
 
-// second pass, one workgroup: counts of all workgroups -> where each workgroup's tokens of an expert start; row and block tables
-__global__ __launch_bounds__(1024) void ob_route_scan_kernel(const ObRouteArgs A, int n_wg)
+// second pass, one workgroup: counts of all workgroups -> where each workgroup's tokens of an expert start; row and block tables.  An expert's
+// workgroups are shared by `runs` threads (runs * experts <= 1024, or one run).
+__global__ __launch_bounds__(1024) void ob_route_scan_kernel(const ObRouteArgs A, int n_wg, int runs)
 {
-    extern __shared__ int icnt[];                                     // [experts]
+    extern __shared__ int icnt[];                                     // [experts] | [runs][experts]
     __shared__ int scan[32];
-    const int tid = threadIdx.x;
+    int *part = icnt + A.experts;
+    const int tid = threadIdx.x, per = (n_wg + runs - 1) / runs;
+    for (int i = tid; i < runs * A.experts; i += 1024) {
+        const int q = i / A.experts, e = i - q * A.experts, b1 = min(n_wg, (q + 1) * per);
+        int c = 0;
+#pragma unroll 4
+        for (int b = q * per; b < b1; ++b) c += A.hist[(size_t)b * A.experts + e];
+        part[i] = c;
+    }
+    __syncthreads();
     for (int e = tid; e < A.experts; e += 1024) {
         int c = 0;
-        for (int b = 0; b < n_wg; b += 8) {
-            int v[8];
-#pragma unroll
-            for (int j = 0; j < 8; ++j) v[j] = A.hist[(size_t)min(b + j, n_wg - 1) * A.experts + e];
-#pragma unroll
-            for (int j = 0; j < 8; ++j)
-                if (b + j < n_wg) { A.hist[(size_t)(b + j) * A.experts + e] = c; c += v[j]; }
-        }
+        for (int q = 0; q < runs; ++q) { const int v = part[q * A.experts + e]; part[q * A.experts + e] = c; c += v; }
         icnt[e] = c;
     }
     __syncthreads();
     ob_route_offsets(A, icnt, scan, tid);
     __syncthreads();
-    for (int e = tid; e < A.experts; e += 1024) {
-        const int r0 = icnt[e];
-        for (int b = 0; b < n_wg; ++b) A.hist[(size_t)b * A.experts + e] += r0;
+    for (int i = tid; i < runs * A.experts; i += 1024) {
+        const int q = i / A.experts, e = i - q * A.experts, b1 = min(n_wg, (q + 1) * per);
+        int c = icnt[e] + part[i];
+        for (int b = q * per; b < b1; ++b) {
+            int *h = A.hist + (size_t)b * A.experts + e;
+            const int v = *h;
+            *h = c;
+            c += v;
+        }
     }
 }
 

@@ -115,6 +115,7 @@ static int dense_heads_launch(ObDenseArgs a, size_t out_step, hipStream_t s)
         a.a = (const char *)a.a + (size_t)OB_SKINNY_T * a.lda * sizeof(E);
         a.u = (char *)a.u + out_step;
         a.act = (char *)a.act + out_step;
+        a.heads = (char *)a.heads + out_step;
     }
     return hstatus("per-head product");
 }
@@ -164,7 +165,7 @@ extern "C" int onebit_hybrid_gemm(const void *w, const void *a, float *z, int32_
 // ----------------------------------------------------------------------------------------------------------- workspace --
 struct HPlan {
     size_t x, emb0, h, u, aux, z, qn, xbc, y, part, ticket, out_h, total;
-    size_t hist, hrm, cq, qu, qa, ctx, lml, kv, actm, actf, acte, acts, ez, route;
+    size_t hist, hrm, cq, qu, qa, ctx, lml, kv, actm, actf, acte, acts, spre, ez, route;
     int64_t kv_rows, ez_rows;
     size_t act[64]; int n_act; int act_mix[64], act_act[64];       // one activation buffer per distinct (mix_k, act_k): its padding stays zero
 };
@@ -174,6 +175,7 @@ static int act_index(const HPlan &P, const onebit_hlayer_t &L)
     return -1;
 }
 #define OB_LAT_PARTS 1024       // (row, split) pairs of the latent decode attention with more than one split
+#define OB_SIDE_SPLITS 4        // K splits of a token input's gate product
 #define OB_EZ_ROWS 4096         // fp32 rows of the experts' partial sums at least
 // rows of the experts' sorted space: every (token, choice), each expert's first row at a multiple of 16
 static int64_t expert_rows(const onebit_hff_t &f, int64_t T) { return T * f.top + 16 * std::min<int64_t>(f.experts, T * f.top); }
@@ -217,7 +219,7 @@ static int make_plan(const onebit_hmodel_t &m, int64_t rows, int64_t n_out, int 
             zc = std::max<int64_t>(zc, 16LL * L.nt_in);
             cq = std::max<int64_t>(cq, R * rup(l.q_rank, kt));
             qu = std::max<int64_t>(qu, R * L.heads * L.kp);
-            qa = std::max<int64_t>(qa, ra * L.heads * l.rp);
+            qa = std::max<int64_t>(qa, ra * rup(L.heads, 16) * l.rp);
             lp = std::max<int64_t>(lp, (int64_t)OB_LAT_PARTS * L.heads * l.rp);
             lml = std::max<int64_t>(lml, 2LL * OB_LAT_PARTS * L.heads);
             if (l.flash) kv = std::max<int64_t>(kv, 2LL * L.heads * P.kv_rows * L.kp);
@@ -255,12 +257,13 @@ static int make_plan(const onebit_hmodel_t &m, int64_t rows, int64_t n_out, int 
     P.actf = take(af * es);
     P.acte = take(ae * es);
     P.acts = take(as * es);
+    P.spre = take((size_t)OB_SIDE_SPLITS * as * 4);
     P.ez = take((size_t)P.ez_rows * (P.ez_rows ? rup(m.width, 16) : 0) * 4);
     P.route = take(rt * 4);
     P.qn = take((size_t)R * qn * es);
     P.xbc = take((size_t)R * xbc * es);
     P.y = take((size_t)R * y * es);
-    P.part = take(std::max<size_t>(max_splits > 1 ? (size_t)max_dec * max_splits * hd * 4 : 0, lp * 4));
+    P.part = take(std::max<size_t>(max_splits > 1 ? (size_t)max_dec * max_splits * hd * 4 : 0, lp * 2));
     P.ticket = take((size_t)max_dec * hd / 128 * 4);
     P.out_h = take((size_t)O * m.width_pad * es);
     P.total = o;
@@ -297,7 +300,8 @@ static int check_model(const onebit_hmodel_t *m)
                     return hfail(ONEBIT_E_SHAPE, "hybrid: layer %d: router sizes", i);
                 ObRouteArgs ra = {};
                 ra.experts = f.experts; ra.identity = f.identity; ra.groups = f.groups;
-                if (ob_route_lds(ra) > 150 * 1024) return hfail(ONEBIT_E_SHAPE, "hybrid: layer %d: too many experts", i);
+                ra.top = f.top;
+                if (n > OB_MOE_MAX || ob_route_lds(ra) > 150 * 1024) return hfail(ONEBIT_E_SHAPE, "hybrid: layer %d: too many experts", i);
             }
             if (L.side.nt < 0 || (L.side.nt & 1) || (L.side.nt && (!L.side.w_gate || !L.side.w_proj || !L.side.norm_w || !L.side.table || L.side.dim <= 0 ||
                                                                     L.side.dim > 16 * L.side.nt || m->side_cols < L.side.dim)))
@@ -353,15 +357,20 @@ template <typename E>
 static int row_launch(const ObXRowArgs &a, int rows, hipStream_t s)
 {
     if (rows <= 0) return 0;
-    const bool ext = a.post_w || a.ez || a.id_w || a.hist || a.out_rm || !a.w || (a.embed && (a.bigram || a.embed_scale != 1.0f));
+    const bool ext = a.post_w || a.top || a.id_w || a.hist || a.out_rm || !a.w || (a.embed && (a.bigram || a.embed_scale != 1.0f));
     const int lds = (((a.W + 3) & ~3) + 16) * 4;
-    const unsigned thr = (unsigned)std::min<int64_t>(rows <= 256 ? 1024 : 512, std::max<int64_t>(64, rup(cdiv(a.W, 4), 64)));
+    const unsigned thr = (unsigned)std::min<int64_t>(rows <= 256 || ext ? 1024 : 512, std::max<int64_t>(64, rup(cdiv(a.W, 4), 64)));
     auto go = [&](auto kern, const auto &args) {
         if (!lds_ok((const void *)kern, lds)) return hfail(ONEBIT_E_SHAPE, "row kernel: LDS");
         hipLaunchKernelGGL(kern, dim3((unsigned)rows), dim3(thr), lds, s, args);
         return hstatus("row kernel");
     };
-    if (ext) return a.W % 4 == 0 ? go(ob_xrow_kernel<E, 4>, a) : go(ob_xrow_kernel<E, 1>, a);
+    if (ext) {
+        const bool one = a.W <= 4 * (int)thr;
+#define OB_XROW(K) (a.W % 4 == 0 ? one ? go(ob_xrow_kernel<E, 4, true, K>, a) : go(ob_xrow_kernel<E, 4, false, K>, a) : go(ob_xrow_kernel<E, 1, false, K>, a))
+        return a.embed ? OB_XROW(OB_X_EMBED) : a.top && a.hist ? OB_XROW(OB_X_BOTH) : a.top ? OB_XROW(OB_X_EXPERTS) : a.hist ? OB_XROW(OB_X_DEPTH) : OB_XROW(OB_X_PLAIN);
+#undef OB_XROW
+    }
     const ObHNormArgs &n = a;
     return a.W % 4 == 0 ? go(ob_hnorm_kernel<E, 4>, n) : go(ob_hnorm_kernel<E, 1>, n);
 }
@@ -530,11 +539,14 @@ static int latent_launch(const onebit_hmodel_t &m, const onebit_hlayer_t &L, con
     if (int rc = part_launch<E>(d, z, n_split, s)) return rc;
     ObLatPrepArgs p = {z, (size_t)T * 16 * L.nt_in, n_split, 16 * L.nt_in, l.q_rank, 16 * l.nt_q, l.kv_rank, l.qn_w, l.kvn_w, m.eps, ws + P.cq, cq_nkt, run.s0, l.rp, bands,
                        st.row_slot, st.row_pos, m.n_slots, m.max_len};
-    const int n_in = l.q_rank + l.kv_rank, plds = (n_in + 16) * 4;
-    auto pk = ob_lat_prep_kernel<E>;
-    if (!lds_ok((const void *)pk, plds)) return hfail(ONEBIT_E_SHAPE, "latent norms: LDS");
-    hipLaunchKernelGGL(pk, dim3((unsigned)T), dim3((unsigned)std::min<int64_t>(T <= 256 ? 1024 : 512, rup(n_in, 64))), plds, s, p);
-    if (int rc = hstatus("latent norms")) return rc;
+    const int n_in = l.q_rank + l.kv_rank, plds = (((n_in + 3) & ~3) + 16) * 4;
+    const bool vec = l.q_rank % 4 == 0 && l.kv_rank % 4 == 0;
+    auto pgo = [&](auto pk) {
+        if (!lds_ok((const void *)pk, plds)) return hfail(ONEBIT_E_SHAPE, "latent norms: LDS");
+        hipLaunchKernelGGL(pk, dim3((unsigned)T), dim3((unsigned)std::min<int64_t>(T <= 256 ? 1024 : 512, rup(cdiv(n_in, vec ? 4 : 1), 64))), plds, s, p);
+        return hstatus("latent norms");
+    };
+    if (int rc = vec ? pgo(ob_lat_prep_kernel<E, 4>) : pgo(ob_lat_prep_kernel<E, 1>)) return rc;
     // queries, row-major [T][H kp]
     ObDenseArgs q = {};
     q.w = l.w_uq; q.a = ws + P.cq; q.n_tiles = q.nt_mix = H * L.kp / 16; q.nkt = cq_nkt; q.T = T; q.u = ws + P.qu;
@@ -548,8 +560,15 @@ static int latent_launch(const onebit_hmodel_t &m, const onebit_hlayer_t &L, con
     if (n_abs) {
         ObDenseArgs k = {};
         k.w = l.w_uk; k.a = ws + P.qu; k.lda = H * L.kp; k.tile_group = l.rp / 16; k.act_cols = L.kp; k.n_tiles = k.nt_mix = H * l.rp / 16; k.nkt = L.kp / KT; k.T = n_abs; k.u = ws + P.qa;
-        if (int rc = dense_heads_launch<E, OB_EPI_IN>(k, (size_t)OB_SKINNY_T * H * l.rp * sizeof(E), s)) return rc;
-        ObLatArgs a = {ws + P.qa, ws + P.ctx, H * l.rp, run.s0, l.rp, bands, st.row_slot, st.row_pos, 0, H, m.n_slots, m.max_len, L.scale, 0, 1, (float *)(ws + P.part), (float *)(ws + P.lml)};
+        if constexpr (sizeof(E) == 2) {
+            if (l.tiled) {
+                k.heads = ws + P.qa; k.head_rows = (int)cdiv(H, 16);
+                for (k.d_shift = 6; (1 << k.d_shift) < l.rp; ++k.d_shift) {}
+                if (int rc = dense_heads_launch<E, OB_EPI_QFRAG>(k, (size_t)OB_SKINNY_T * rup(H, 16) * l.rp * sizeof(E), s)) return rc;
+            }
+        }
+        if (!l.tiled) if (int rc = dense_heads_launch<E, OB_EPI_IN>(k, (size_t)OB_SKINNY_T * H * l.rp * sizeof(E), s)) return rc;
+        ObLatArgs a = {ws + P.qa, ws + P.ctx, H * l.rp, run.s0, l.rp, bands, st.row_slot, st.row_pos, 0, H, m.n_slots, m.max_len, L.scale, 0, 1, ws + P.part, (float *)(ws + P.lml)};
         if (!l.tiled) {
             auto rk = ob_lat_rows_kernel<E>;
             const int lds = (l.rp + 256 + 16) * 4;
@@ -563,8 +582,11 @@ static int latent_launch(const onebit_hmodel_t &m, const onebit_hlayer_t &L, con
             if (st.n_dec || st.n_short) ctx = st.attn_chunk * st.attn_splits;
             for (int i = st.n_short; i < (first == st.n_seg ? st.n_seg : 0); ++i) ctx = std::max(ctx, st.segs[i].past + st.segs[i].n);
             const int ht = H > 16 && l.rp <= 512 ? 2 : 1, hg = (int)cdiv(H, 16 * ht);
-            const int64_t want = std::min<int64_t>({512 / ((int64_t)n_abs * hg), cdiv(ctx, 128), OB_LAT_PARTS / n_abs});
-            a.chunk = (int)rup(cdiv(ctx, std::max<int64_t>(1, want)), 128);
+            // one round of workgroups (two thirds of the LDS each at 512 columns); a split writes and the combining launch reads all heads' outputs
+            // in fp32, so never more splits than that needs, and at most 32
+            const int per_cu = l.rp >= 512 ? 1 : l.rp >= 256 ? 2 : 4;
+            const int64_t want = std::min<int64_t>({256 * per_cu / ((int64_t)n_abs * hg), cdiv(ctx, 64), OB_LAT_PARTS / n_abs, 32});
+            a.chunk = (int)rup(cdiv(ctx, std::max<int64_t>(1, want)), 64);
             a.nsplit = (int)cdiv(ctx, a.chunk);
             for (int r0 = 0; r0 < n_abs; r0 += 32768) {
                 a.row0 = r0;
@@ -572,7 +594,7 @@ static int latent_launch(const onebit_hmodel_t &m, const onebit_hlayer_t &L, con
                 auto go = [&](auto kern, int rp) {
                     const int lds = 2 * rp * 128 + 16 * ht * 68 * 4;
                     if (!lds_ok((const void *)kern, lds)) return hfail(ONEBIT_E_SHAPE, "latent attention: LDS");
-                    hipLaunchKernelGGL(kern, grid, dim3(256), lds, s, a);
+                    hipLaunchKernelGGL(kern, grid, dim3(256 * ht), lds, s, a);
                     return hstatus("latent attention");
                 };
                 int rc;
@@ -583,7 +605,7 @@ static int latent_launch(const onebit_hmodel_t &m, const onebit_hlayer_t &L, con
                             : l.rp == 256 ? go(ob_lat_dec_kernel<256, 1>, 256) : go(ob_lat_dec_kernel<512, 1>, 512);
                 } else rc = hfail(ONEBIT_E_DTYPE, "latent attention: tiled form in fp32");
                 if (rc) return rc;
-                if (a.nsplit > 1) hipLaunchKernelGGL(ob_lat_combine_kernel, dim3((unsigned)H, grid.y), dim3((unsigned)std::min<int64_t>(256, rup(l.rp / 4, 64))), 0, s, a);
+                if (a.nsplit > 1) hipLaunchKernelGGL(ob_lat_combine_kernel, dim3((unsigned)H, grid.y), dim3((unsigned)std::min<int64_t>(256, rup(l.rp / 8, 64))), 0, s, a);
             }
         }
         if (int rc = hstatus("latent attention")) return rc;
@@ -685,16 +707,18 @@ static int ff_launch(const onebit_hmodel_t &m, const onebit_hlayer_t &L, const o
     r.gather = at; at += S;
     r.hist = at;
     r.block_rows = br; r.n_blk = n_blk;
-    const int lds = (int)ob_route_lds(r);
-    if (n_wg == 1) {
-        auto k = ob_route_kernel<true>;
-        if (!lds_ok((const void *)k, lds)) return hfail(ONEBIT_E_SHAPE, "router: LDS");
-        hipLaunchKernelGGL(k, dim3(1), dim3(1024), lds, s, r);
-    } else {
-        auto k = ob_route_kernel<false>;
+    const int lds = (int)ob_route_lds(r), n_all = f.experts + f.identity;
+    auto route = [&](auto k) {
         if (!lds_ok((const void *)k, lds)) return hfail(ONEBIT_E_SHAPE, "router: LDS");
         hipLaunchKernelGGL(k, dim3((unsigned)n_wg), dim3(1024), lds, s, r);
-        hipLaunchKernelGGL(ob_route_scan_kernel, dim3(1), dim3(1024), f.experts * 4, s, r, n_wg);
+        return 0;
+    };
+#define OB_ROUTE(S) (n_all <= 64 ? route(ob_route_kernel<S, 1>) : n_all <= 256 ? route(ob_route_kernel<S, 4>) : route(ob_route_kernel<S, 16>))
+    if (int rc = n_wg == 1 ? OB_ROUTE(true) : OB_ROUTE(false)) return rc;
+#undef OB_ROUTE
+    if (n_wg > 1) {
+        const int runs = std::max(1, 1024 / f.experts);
+        hipLaunchKernelGGL(ob_route_scan_kernel, dim3(1), dim3(1024), f.experts * 4 * (runs + 1), s, r, n_wg, runs);
         hipLaunchKernelGGL(ob_route_rows_kernel, dim3((unsigned)n_wg), dim3(256), f.experts * 4, s, r);
     }
     if (int rc = hstatus("router")) return rc;
@@ -708,13 +732,54 @@ static int ff_launch(const onebit_hmodel_t &m, const onebit_hlayer_t &L, const o
     int n_split = 1;
     if (br == OB_SKINNY_T) n_split = (int)std::max<int64_t>(1, std::min<int64_t>({cdiv(512, cdiv(wt, 2) * live), o.nkt / 8, OB_EZ_ROWS / S, 8}));
     n_split = (int)cdiv(o.nkt, cdiv(o.nkt, n_split));
-    if (int rc = dense_blocks_launch<E, OB_EPI_PART, OB_ROWS_SORTED>(o, n_blk, br, n_split, s)) return rc;
-    pend.ez = o.z; pend.ez_split = o.z_split; pend.ez_n = n_split; pend.ld_ez = o.ldz; pend.top = f.top; pend.tok_row = r.tok_row; pend.tok_w = r.tok_w;
+    if (br == OB_SKINNY_T) {
+        if (int rc = dense_blocks_launch<E, OB_EPI_PART, OB_ROWS_SORTED>(o, n_blk, br, n_split, s)) return rc;
+        pend.ez = o.z;
+    } else {                                                          // many rows: outputs in the work type, half the traffic
+        o.u = o.z; o.nt_mix = wt;
+        if (int rc = dense_blocks_launch<E, OB_EPI_IN, OB_ROWS_SORTED>(o, n_blk, br, 1, s)) return rc;
+        pend.eo = o.u;
+    }
+    pend.ez_split = o.z_split; pend.ez_n = n_split; pend.ld_ez = o.ldz; pend.top = f.top; pend.tok_row = r.tok_row; pend.tok_w = r.tok_w;
     if (f.identity) {
         pend.id_w = r.id_w;
         if (L.pre2_w) { pend.idh = ws + P.hrm; pend.ld_idh = m.width_pad; }
     }
     return 0;
+}
+
+// the token's own input: gate product, gelu and the token's row, output product
+template <typename E>
+static int side_launch(const onebit_hmodel_t &m, const onebit_hlayer_t &L, const onebit_hstate_t &st, const HPlan &P, char *ws, int &n_split, hipStream_t s)
+{
+    constexpr int KT = ObElem<E>::KT;
+    const int T = st.n_rows, nkt = 16 * L.side.nt / KT;
+    ObDenseArgs g = {}, o = {};
+    g.w = L.side.w_gate; g.a = ws + P.h; g.n_tiles = L.side.nt; g.nkt = m.width_pad / KT; g.T = T;
+    o.w = L.side.w_proj; o.n_tiles = (int)cdiv(m.width, 16); o.nkt = nkt; o.T = T;
+    o.table = L.side.table; o.ld_table = m.side_cols; o.table_cols = L.side.dim; o.tokens = st.tokens;
+    float *pre = (float *)(ws + P.spre);
+    g.z = pre; g.ldz = 16 * L.side.nt; g.z_split = (size_t)T * g.ldz;
+    const int64_t wgs = T <= OB_SKINNY_T ? cdiv(g.n_tiles, 2) : cdiv(g.n_tiles, 8) * cdiv(T, 128);
+    int n_pre = (int)std::max<int64_t>(1, std::min<int64_t>({cdiv(512, wgs), g.nkt / 16, OB_SIDE_SPLITS}));
+    n_pre = (int)cdiv(g.nkt, cdiv(g.nkt, n_pre));
+    if (int rc = dense_launch<E, OB_EPI_PART>(g, n_pre, s)) return rc;
+    o.pre = pre; o.n_pre = n_pre; o.ld_pre = g.ldz;
+    const int mt = T <= 16 ? 1 : T <= 32 ? 2 : 4, lds = mt * nkt * 1024;
+    if (T <= OB_SKINNY_T && lds <= 48 * 1024) {                       // few rows: the output product forms its own operand
+        o.z = (float *)(ws + P.z); o.ldz = 16 * o.n_tiles; o.z_split = (size_t)T * o.ldz; o.kt_split = o.nkt;
+        n_split = 1;
+        const dim3 grid((unsigned)cdiv(o.n_tiles, 2));
+        if (mt == 1) hipLaunchKernelGGL((ob_dense_skinny_kernel<E, OB_EPI_PART, 1, OB_ROWS_TABLE>), grid, dim3(256), lds, s, o);
+        else if (mt == 2) hipLaunchKernelGGL((ob_dense_skinny_kernel<E, OB_EPI_PART, 2, OB_ROWS_TABLE>), grid, dim3(256), lds, s, o);
+        else hipLaunchKernelGGL((ob_dense_skinny_kernel<E, OB_EPI_PART, 4, OB_ROWS_TABLE>), grid, dim3(256), lds, s, o);
+        return hstatus("token input");
+    }
+    o.act = ws + P.acts;
+    hipLaunchKernelGGL(ob_table_rows_kernel<E>, dim3((unsigned)cdiv((int64_t)T * nkt * KT / 4, 256)), dim3(256), 0, s, o);
+    if (int rc = hstatus("token input")) return rc;
+    o.a = o.act;
+    return part_launch<E>(o, (float *)(ws + P.z), n_split, s);
 }
 
 template <typename E>
@@ -791,15 +856,10 @@ static int step_impl(const onebit_hmodel_t &m, const onebit_hstate_t &st, const 
                 a = pend;
                 a.w = nullptr; a.out = ws + P.h;
                 if (int rc = row_launch<E>(a, T, s)) return rc;
-                ObDenseArgs g = {};
-                g.w = L.side.w_gate; g.a = ws + P.h; g.n_tiles = L.side.nt; g.nkt = w_nkt; g.T = T; g.act = ws + P.acts; g.act_nkt = 16 * L.side.nt / KT;
-                g.fn = OB_FN_GELU_TABLE; g.table = L.side.table; g.ld_table = m.side_cols; g.table_cols = L.side.dim; g.tokens = st.tokens;
-                if (int rc = dense_launch<E, OB_EPI_ACT>(g, 1, s)) return rc;
-                o.w = L.side.w_proj; o.a = g.act; o.nkt = g.act_nkt;
                 pend = nb;
                 pend.mult = 1.0f;
                 pend.z = (float *)(ws + P.z); pend.z_split = (size_t)T * ldz; pend.post_w = L.side.norm_w;
-                if (int rc = part_launch<E>(o, (float *)(ws + P.z), pend.n_split, s)) return rc;
+                if (int rc = side_launch<E>(m, L, st, P, ws, pend.n_split, s)) return rc;
             }
         }
         keep_result(r + 1, L.dwa);

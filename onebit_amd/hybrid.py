@@ -444,8 +444,9 @@ class HybridDecoder:
             d = layers[i].depth_average
             if d is not None and d.shape != (r + 2,):
                 raise ValueError(f"layer run {r}: a depth average over {tuple(d.shape)} of {r + 2} results")
-        self.embed_scale, self.bigram_mul = float(embed_scale), tuple(int(v) for v in bigram_mul)
+        self.embed_scale = float(embed_scale)
         self.bigram = None if bigram is None else bigram.to(dtype).contiguous()
+        self.bigram_mul = (0, 0) if bigram is None else tuple(int(v) % (bigram.shape[0] - 1) for v in bigram_mul)      # (the row is taken modulo the buckets)
         self.embed = embed.to(dtype).contiguous()
         self.pos_embed = None if pos_embed is None else pos_embed.to(dtype).contiguous()
         self.final_norm = final_norm.float().contiguous()

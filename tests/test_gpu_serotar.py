@@ -207,7 +207,7 @@ def test_router_details_show(dtype):
 @DTYPES
 def test_embedding_alone(dtype):
     """Scale and bigram rows; the previous token comes from the slot when a portion or a decoded token starts behind it."""
-    raw = raw_config([layer(None)], width=50, vocab=90, scale=2.25, bigram=(31, 1000003, 77777))
+    raw = raw_config([layer(None)], width=50, vocab=90, scale=2.25, bigram=(31, 5000000029, 77777))
 
     def edit(w):
         only()(w)
@@ -219,7 +219,7 @@ def test_embedding_alone(dtype):
         assert err(run_cut(eng, 1, toks, cuts), ref) < TOL[dtype], cuts
     other = tokens(40, 90, 5)                                                  # the slot again: the first token's row does not look back
     assert err(run_cut(eng, 1, other, [30]), R.forward(raw, w, other)) < TOL[dtype]
-    swapped = R.forward(dict(raw, embedding=dict(raw["embedding"], bigram=dict(buckets=31, mul_prev=77777, mul_cur=1000003))), w, toks)
+    swapped = R.forward(dict(raw, embedding=dict(raw["embedding"], bigram=dict(buckets=31, mul_prev=77777, mul_cur=5000000029))), w, toks)
     assert err(swapped, ref) > 0.2
 
 
