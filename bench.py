@@ -91,7 +91,7 @@ def serotar_config(width, layers=8, vocab=32000):
     h, d, qr, kr, side = SEROTAR_SIZES[width]
     mix = {"heads": h, "dim": d, "vdim": d, "q_rank": qr, "kv_rank": kr, "scale": d ** -0.5}
     moe = {"kind": "moe", "expert": {"ff": ff // 8}, "shared": {"ff": ff // 4}, "router": {"experts": 32, "identity": 8, "top": 6, "groups": {"count": 8, "keep": 4}}}
-    return SerotarConfig(vocab_size=vocab, width=width, norm_eps=1e-5, embed_scale=1.0, bigram={"buckets": 4 * vocab - 1, "mul_prev": 31, "mul_cur": 7}, side_dim=side,
+    return SerotarConfig(vocab_size=vocab, width=width, norm_eps=1e-5, embed_scale=1.0, bigram={"buckets": 4 * vocab - 1, "mul_prev": 53, "mul_cur": 11}, side_dim=side,
                          layers=[{"type": "latent_attention", "mixer": mix, "mlp": moe if i else {"kind": "dense", "ff": ff}} for i in range(layers)])
 
 

@@ -582,8 +582,8 @@ static int latent_launch(const onebit_hmodel_t &m, const onebit_hlayer_t &L, con
             if (st.n_dec || st.n_short) ctx = st.attn_chunk * st.attn_splits;
             for (int i = st.n_short; i < (first == st.n_seg ? st.n_seg : 0); ++i) ctx = std::max(ctx, st.segs[i].past + st.segs[i].n);
             const int ht = H > 16 && l.rp <= 512 ? 2 : 1, hg = (int)cdiv(H, 16 * ht);
-            // one round of workgroups (two thirds of the LDS each at 512 columns); a split writes and the combining launch reads all heads' outputs
-            // in fp32, so never more splits than that needs, and at most 32
+            // as many workgroups as run at once (their LDS decides: one per CU at 512 columns); every split writes all heads' outputs for the
+            // combining launch to read, so never more than that, and at most 32
             const int per_cu = l.rp >= 512 ? 1 : l.rp >= 256 ? 2 : 4;
             const int64_t want = std::min<int64_t>({256 * per_cu / ((int64_t)n_abs * hg), cdiv(ctx, 64), OB_LAT_PARTS / n_abs, 32});
             a.chunk = (int)rup(cdiv(ctx, std::max<int64_t>(1, want)), 64);

@@ -101,7 +101,7 @@ def only(*keep):
 
 
 # ------------------------------------------------------------------------------------------------- each mechanism alone --
-ATTENTION_SIZES = [dict(heads=4, dim=64, vdim=64, q_rank=80, kv_rank=128, scale=0.125), dict(heads=3, dim=24, vdim=40, q_rank=20, kv_rank=36, scale=0.4),
+ATTENTION_SIZES = [dict(heads=6, dim=64, vdim=56, q_rank=72, kv_rank=112, scale=0.14), dict(heads=3, dim=24, vdim=40, q_rank=20, kv_rank=36, scale=0.4),
                    dict(heads=17, dim=16, vdim=80, q_rank=50, kv_rank=200, scale=0.3), dict(heads=33, dim=100, vdim=128, q_rank=33, kv_rank=64, scale=0.1),
                    dict(heads=1, dim=1, vdim=3, q_rank=2, kv_rank=5, scale=1.0), dict(heads=2, dim=144, vdim=136, q_rank=64, kv_rank=300, scale=0.08),
                    dict(heads=20, dim=128, vdim=64, q_rank=96, kv_rank=512, scale=0.09), dict(heads=2, dim=32, vdim=48, q_rank=40, kv_rank=530, scale=0.2)]
@@ -135,7 +135,7 @@ def test_xielu_feed_forward_alone(ff, dtype):
             assert err(run(m.step_engine(1, 256), 0, 0, toks), R.forward(raw, w, toks)) < TOL[dtype], (p, T)
 
 
-MIXTURES = {"as-named": moe(8, 3, 4, (3, 2), 64, 128), "no-identity-no-groups": moe(5, 2, 0, None, 24, 0), "mostly-identity": moe(2, 3, 10, (4, 3), 17, 9),
+MIXTURES = {"plain": moe(10, 3, 5, (5, 3), 56, 96), "no-identity-no-groups": moe(5, 2, 0, None, 24, 0), "mostly-identity": moe(2, 3, 10, (4, 3), 17, 9),
             "one-of-many": moe(40, 1, 0, (8, 1), 16, 48), "all": moe(3, 4, 1, (2, 2), 40, 0), "one-expert": moe(1, 1, 0, None, 33, 0), "wide-group": moe(70, 9, 58, (2, 1), 8, 8)}
 
 
@@ -318,7 +318,7 @@ def test_sequential_layers_of_other_mixers(dtype):
 
 # ------------------------------------------------------------------------------------------------------ whole models --
 MODELS = {
-    "mixed": raw_config([layer(dense(56)), layer(moe(8, 2, 2, (5, 3), 24, 40)), layer(moe(5, 2, 1, (3, 2), 40, 0), heads=2, dim=32, vdim=48, kv_rank=70)], width=64, vocab=150),
+    "mixed": raw_config([layer(dense(56)), layer(moe(9, 2, 1, (5, 3), 24, 40)), layer(moe(5, 2, 1, (3, 2), 40, 0), heads=2, dim=32, vdim=48, kv_rank=70)], width=64, vocab=150),
     "odd": raw_config([layer(moe(3, 1, 2, None, 11, 13), heads=5, dim=9, vdim=7, q_rank=13, kv_rank=21, scale=0.6), layer(None), layer(dense(29), heads=1, dim=70, vdim=90, kv_rank=130)],
                       width=50, vocab=77, side=29, bigram=(11, 2, 3)),
     "bare": raw_config([layer(dense(40)), layer(dense(24), heads=4, dim=64, vdim=32, q_rank=48, kv_rank=96, scale=0.1)], width=80, vocab=90, side=0, bigram=None),
@@ -421,6 +421,34 @@ def test_many_requests_and_expansion_in_groups(zoo, dtype):
         alone.append(run(eng, s, 900 + s, far[900 + s:925 + s]))
     eng.launch([(s, 900 + s, far[900 + s:925 + s], list(range(25))) for s in range(6)])
     assert err(eng.logits[:150], torch.cat(alone).cpu()) < (0.02 if dtype == BF else 1e-5)
+
+
+@pytest.mark.parametrize("seed", range(6))
+def test_random_sizes(seed):
+    """Layers of random kinds and sizes in fp32: whole, and in random portions."""
+    import random
+    rg = random.Random(seed)
+
+    def lay():
+        m = dict(heads=rg.randint(1, 20), dim=rg.choice([8, 12, 24, 48, 80, 136]), vdim=rg.choice([8, 20, 32, 72, 96, 144]), q_rank=rg.choice([17, 32, 60, 96]),
+                 kv_rank=rg.choice([24, 50, 96, 160, 256, 520]))
+        kind = rg.randrange(3)
+        if kind == 0:
+            return layer(None if rg.random() < 0.3 else dense(rg.choice([7, 32, 100])), scale=m["dim"] ** -0.5, **m)
+        experts, identity = rg.randint(2, 20), rg.choice([0, 1, 4, 6])
+        counts = [c for c in range(1, experts + identity) if (experts + identity) % c == 0]
+        count = rg.choice(counts)
+        keep = rg.randint(1, count)
+        return layer(moe(experts, rg.randint(1, min(6, keep * ((experts + identity) // count))), identity, (count, keep), rg.choice([8, 17, 64]), rg.choice([0, 24, 100])),
+                     scale=m["dim"] ** -0.5, **m)
+    raw = raw_config([lay() for _ in range(rg.randint(1, 4))], width=rg.choice([48, 50, 100, 192]), vocab=rg.choice([61, 100, 300]), side=rg.choice([0, 18, 33]),
+                     bigram=rg.choice([None, (101, 19, 11)]))
+    m, w = build(raw, F32, seed=seed)
+    toks = tokens(150, raw["vocab"], seed)
+    ref, eng, cuts = R.forward(raw, w, toks), m.step_engine(3, 200), []
+    while sum(cuts) < 140:
+        cuts.append(min(142 - sum(cuts), rg.choice([1, 2, 5, 16, 17, 40, 64])))
+    assert err(run(eng, 0, 0, toks), ref) < TOL[F32] and err(run_cut(eng, 1, toks, cuts), ref) < TOL[F32], (raw, cuts)
 
 
 @DTYPES
